@@ -52,9 +52,11 @@ class LayerSpec:
 @dataclass(frozen=True)
 class ScheduleEntry:
     """One run of a layer.  ``cache_of`` names an earlier entry whose cache this run reads
-    instead of keeping its own."""
+    instead of keeping its own.  ``step_vector`` t: row t of the model's step vectors is added to the residual stream of
+    every token before this run."""
     layer: int
     cache_of: int | None = None
+    step_vector: int | None = None
 
 
 @dataclass
@@ -74,6 +76,9 @@ class ModelPlan:
     logit_scale: float = 1.0                # the logits are multiplied by it, before the cap
     position_table: Source | None = None    # a learned vector per position [max_positions, H], added to the embedded token
 
+    step_vectors: Source | None = None      # a vector per pass of a loop [n_step_vectors, H]: see ScheduleEntry.step_vector
+    n_step_vectors: int = 0
+
     def validate(self) -> None:
         n = len(self.layers)
         if self.logit_softcap is not None and not self.logit_softcap > 0:
@@ -83,3 +88,5 @@ class ModelPlan:
                 raise ValueError(f"schedule entry {i} names layer {e.layer}, model has {n}")
             if e.cache_of is not None and not 0 <= e.cache_of < i:
                 raise ValueError(f"schedule entry {i} reads the cache of entry {e.cache_of}, which does not run before it")
+            if e.step_vector is not None and not (self.step_vectors is not None and 0 <= e.step_vector < self.n_step_vectors):
+                raise ValueError(f"schedule entry {i} adds step vector {e.step_vector}, the model has {self.n_step_vectors}")

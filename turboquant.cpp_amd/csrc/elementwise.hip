@@ -246,6 +246,155 @@ TQ_API int tq_add_rmsnorm(float* x, const float* delta, int S, int64_t delta_str
   return 0;
 }
 
+// ---------------------------------------------------------------- residual sum of several parts + RMS norm
+// As add_rmsnorm, for arrangements whose parts run side by side: what is added to x[row] is
+//   vec[:]                                                (a vector that is the same for every row; null: none)
+//   + sum_j weights[row][j] * y[pair_slot[row][j]]        (the experts' unsummed rows; y null: none)
+//   + sum_g coef[g] * sum_s delta_g[s][row]               (up to TERMS parts, each S[g] partial sums delta_stride apart)
+// in that order, and the sum is normed: out = (v * (1/sqrt(mean v^2 + eps))) * w.  w null: the stream is summed and nothing
+// is returned.
+#define TERMS 4
+#define TERM_SLICES 128      // partial sums of all parts together
+struct TermArgs {
+  const float* delta[TERMS];
+  int S[TERMS];
+  float coef[TERMS];
+  int n;
+};
+
+template <class W>
+__global__ void add_terms_rmsnorm_kernel(float* __restrict__ x, TermArgs terms, size_t delta_stride, const float* __restrict__ vec,
+                                         const float* __restrict__ y, const int* __restrict__ pair_slot,
+                                         const float* __restrict__ weights, int topk, const W* __restrict__ w, float eps,
+                                         const int* __restrict__ rows, act_t* __restrict__ out, float* __restrict__ out32, int H) {
+  extern __shared__ __attribute__((aligned(16))) float v[];       // H floats, then one float per wave
+  __shared__ int slot[64];
+  __shared__ float wgt[64];
+  __shared__ const float* src[TERM_SLICES];
+  __shared__ float cf[TERM_SLICES];
+  float* red = v + (H + 3) / 4 * 4;
+  const int r = blockIdx.x;
+  const int row = rows ? rows[r] : r;
+  float* xr = x + (size_t)row * H;
+  int N = 0;
+#pragma unroll
+  for (int g = 0; g < TERMS; ++g) {
+    if (g < terms.n) {
+      if ((int)threadIdx.x < terms.S[g]) {
+        src[N + threadIdx.x] = terms.delta[g] + threadIdx.x * delta_stride + (size_t)row * H;
+        cf[N + threadIdx.x] = terms.coef[g];
+      }
+      N += terms.S[g];
+    }
+  }
+  if (y && (int)threadIdx.x < topk) {
+    slot[threadIdx.x] = pair_slot[(size_t)row * topk + threadIdx.x];
+    wgt[threadIdx.x] = weights[(size_t)row * topk + threadIdx.x];
+  }
+  __syncthreads();
+  float ss = 0.f;
+  if (H % 4 == 0) {
+#pragma unroll 2
+    for (int i = threadIdx.x * 4; i < H; i += blockDim.x * 4) {
+      f32x4 a = load4f(xr + i);
+      if (vec) a += load4f(vec + i);
+      if (y) {
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j < topk; j += 4) {
+          f32x4 t[4];
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            if (j + u < topk) t[u] = slot[j + u] < 0 ? f32x4{0.f, 0.f, 0.f, 0.f} : load4f(y + (size_t)slot[j + u] * H + i);
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            if (j + u < topk) acc += wgt[j + u] * t[u];
+        }
+        a += acc;
+      }
+      for (int s = 0; s < N; s += 4) {
+        f32x4 t[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (s + u < N) t[u] = load4f(src[s + u] + i);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (s + u < N) a += cf[s + u] * t[u];
+      }
+      store4(v + i, a);
+      if (!rows) store4(xr + i, a);
+      ss += a.x * a.x;
+      ss += a.y * a.y;
+      ss += a.z * a.z;
+      ss += a.w * a.w;
+    }
+  } else {
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      float a = xr[i];
+      if (vec) a += vec[i];
+      if (y) {
+        float acc = 0.f;
+        for (int j = 0; j < topk; ++j)
+          if (slot[j] >= 0) acc += wgt[j] * y[(size_t)slot[j] * H + i];
+        a += acc;
+      }
+      for (int s = 0; s < N; ++s) a += cf[s] * src[s][i];
+      v[i] = a;
+      if (!rows) xr[i] = a;
+      ss += a * a;
+    }
+  }
+  if (!w) return;
+  ss = block_sum(ss, red);
+  const float rs = 1.0f / sqrtf(ss / (float)H + eps);
+  if (H % 4 == 0) {
+#pragma unroll 2
+    for (int i = threadIdx.x * 4; i < H; i += blockDim.x * 4) {
+      const f32x4 o = load4f(v + i) * rs * load4f(w + i);
+      if (out) store4(out + (size_t)r * H + i, o);
+      if (out32) store4(out32 + (size_t)r * H + i, o);
+    }
+  } else {
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      const float o = v[i] * rs * to_f32(w[i]);
+      if (out) out[(size_t)r * H + i] = from_f32<act_t>(o);
+      if (out32) out32[(size_t)r * H + i] = o;
+    }
+  }
+}
+
+// deltas, S, coef: n parts (host arrays; n may be 0), all with partial sums delta_stride floats apart.
+TQ_API int tq_add_terms_rmsnorm(float* x, const int64_t* deltas, const int* S, const float* coef, int n, int64_t delta_stride,
+                                const float* vec, const float* y, const int* pair_slot, const float* weights, int topk,
+                                const void* w, int wtype, float eps, const int* rows, int R, void* out, float* out32, int H,
+                                hipStream_t st) {
+  if (R <= 0) return 0;
+  if (n < 0 || n > TERMS) return TQ_ERR_UNSUPPORTED;
+  if (y && (topk < 1 || topk > 64 || !pair_slot || !weights)) return TQ_ERR_BAD_ARG;
+  if (!w && (rows || out || out32)) return TQ_ERR_BAD_ARG;
+  TermArgs t{};
+  int slices = 0;
+  for (int g = 0; g < n; ++g) {
+    if (!deltas[g] || S[g] < 1) return TQ_ERR_BAD_ARG;
+    t.delta[g] = (const float*)(uintptr_t)deltas[g];
+    t.S[g] = S[g];
+    t.coef[g] = coef[g];
+    slices += S[g];
+  }
+  t.n = n;
+  if (slices > TERM_SLICES) return TQ_ERR_UNSUPPORTED;
+  const int threads = (H % 4 == 0 && H >= 2048) ? 512 : 256;
+  const size_t shmem = (size_t)((H + 3) / 4 * 4 + threads / TQ_WAVE) * sizeof(float);
+  if (shmem > 150 * 1024) return TQ_ERR_UNSUPPORTED;
+  TQ_DISPATCH_W(wtype, {
+    if (shmem > 48 * 1024)
+      (void)hipFuncSetAttribute((const void*)add_terms_rmsnorm_kernel<W>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem);
+    hipLaunchKernelGGL(add_terms_rmsnorm_kernel<W>, dim3(R), dim3(threads), shmem, st, x, t, (size_t)delta_stride, vec, y,
+                       pair_slot, weights, topk, (const W*)w, eps, rows, (act_t*)out, out32, H);
+  });
+  TQ_LAUNCH_CHECK();
+  return 0;
+}
+
 // The limit of gated pairs that the next launches of products and of gated_act take (common.h: gated_pair); 0: none.
 float tq_pair_limit_host = 0.f;
 TQ_API int tq_set_pair_limit(float limit) {

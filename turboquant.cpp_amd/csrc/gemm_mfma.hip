@@ -22,6 +22,7 @@
 #include "common.h"
 
 #include "gemm_mfma.h"
+#include <string.h>
 
 // ------------------------------------------------------------------------------------------ few rows
 // The sums of one wave: its share k_beg .. k_end of k for NTL tiles of 16 columns (tile t starts at column col0[t])
@@ -949,8 +950,8 @@ TQ_API int tq_gemm_mfma_pair_splits(int N1, int K1, int grouped1, int N2, int K2
   return (K2 + k_per - 1) / k_per;
 }
 
-// Two products of few rows in one launch.  d1, d2: 19 numbers each, in the order of tq_gemm_mfma's arguments from
-// `a` to `tile_rows`, then the gate's activation.  Both must be products that the streaming kernel takes 16 rows at a time (a matrix per
+// Two products of few rows in one launch.  d1, d2: 20 numbers each, in the order of tq_gemm_mfma's arguments from
+// `a` to `tile_rows`, then the gate's activation and the bits of the gated pair's limit as a float (0: none).  Both must be products that the streaming kernel takes 16 rows at a time (a matrix per
 // expert with tile_rows 16, or one matrix with M <= 16), both gated or both not, both into the same type.  The
 // waves that split k are those of the first product (the larger one by convention).  splits2 > 1 (as
 // tq_gemm_mfma_pair_splits says, for a plain second product into float): run z of its k goes to
@@ -967,7 +968,10 @@ TQ_API int tq_gemm_mfma_pair(const int64_t* d1, const int64_t* d2, int splits2, 
     if (((uintptr_t)p[0] | (uintptr_t)p[4] | (uintptr_t)p[5]) % 16 != 0) return TQ_ERR_BAD_ARG;
     g[i] = MfmaGemmArgs{(const bf16_t*)p[0], p[1], (const int*)p[2], (int)p[3], (const bf16_t*)p[4], (const bf16_t*)p[5],
                         p[6], (const int*)p[7], (const int*)p[8], (const void*)p[9], (int)p[10], (void*)p[11], p[12],
-                        M, N, K, K, 0, (int)p[18], 1, 0, tq_pair_limit_host};
+                        M, N, K, K, 0, (int)p[18], 1, 0, 0.f};
+    const uint32_t limit_bits = (uint32_t)p[19];
+    memcpy(&g[i].limit, &limit_bits, sizeof(float));
+    if (!(g[i].limit >= 0.f)) return TQ_ERR_BAD_ARG;
     if (g[i].gate < 0 || g[i].gate >= TQ_GATE_COUNT) return TQ_ERR_BAD_ARG;
     dual[i] = p[5] != 0;
     out_act[i] = p[13] != 0;

@@ -204,10 +204,10 @@ int product(Ctx& c, const Product& p, void** out, int* splits, int side = 0) {
 
 #if defined(TQ_ACT_BF16)
 void pair_desc(const Product& p, void* out, int tile_rows, int64_t* d) {
-  const int64_t v[19] = {(int64_t)(uintptr_t)p.a, p.lda, (int64_t)(uintptr_t)p.a_rows, p.gather, (int64_t)(uintptr_t)p.w.ptr,
+  const int64_t v[20] = {(int64_t)(uintptr_t)p.a, p.lda, (int64_t)(uintptr_t)p.a_rows, p.gather, (int64_t)(uintptr_t)p.w.ptr,
                          (int64_t)(uintptr_t)p.w2, p.gstride, (int64_t)(uintptr_t)p.tile_group, (int64_t)(uintptr_t)p.n_tiles,
                          (int64_t)(uintptr_t)p.bias.ptr, p.bias.ptr ? p.bias.wtype : 0, (int64_t)(uintptr_t)out, p.N, p.out_act,
-                         p.M, p.N, p.K, tile_rows, p.gate};
+                         p.M, p.N, p.K, tile_rows, p.gate, 0};
   memcpy(d, v, sizeof(v));
 }
 #endif
@@ -230,7 +230,7 @@ int product_pair(Ctx& c, const Product& p1, const Product& p2, void** out1, void
     if (p2.partial) *splits2 = tq_gemm_mfma_pair_splits(p1.N, p1.K, p1.tile_group != nullptr, p2.N, p2.K, 0);
     *out1 = c.arena.take((size_t)p1.M * p1.N * (p1.out_act ? TQ_ACT_BYTES : 4));
     *out2 = c.arena.take((size_t)*splits2 * p2.M * p2.N * (p2.out_act ? TQ_ACT_BYTES : 4));
-    int64_t d1[19], d2[19];
+    int64_t d1[20], d2[20];
     pair_desc(p1, *out1, tile_rows[0], d1);
     pair_desc(p2, *out2, tile_rows[1], d2);
     RUN(c, "gemm_pair", tq_gemm_mfma_pair(d1, d2, *splits2, c.stream));

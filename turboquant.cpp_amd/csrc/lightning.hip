@@ -17,13 +17,16 @@
 //                   silu applied as they are staged.  The order of every sum depends on the sizes only, never on how
 //                   the sequence was cut into steps or on what else the step holds.
 //   lightning_out   per token: the norm over all heads, the weight and the gate, into the activation type.
-#include "common.h"
+#include "linear_chunks.h"
 
 #define LN_ROWS 16        // key channels of a value channel that one lane keeps
 #define LN_CHUNK 16       // tokens staged at a time
 #define LN_SEG 20         // floats between the rows of two lanes in LDS (16 would put eight lanes on four banks)
 
 __device__ __forceinline__ float ln_silu(float x) { return x / (1.0f + expf(-x)); }
+struct LnSilu {
+  __device__ __forceinline__ float operator()(float x) const { return ln_silu(x); }
+};
 
 // grid (ceil(V / VB), H, B), block 256; L = lanes per value channel (a power of two, L * LN_ROWS >= D), VB = 256 / L.
 template <int L>
@@ -126,57 +129,6 @@ TQ_API int tq_lightning_scan(const float* P, int64_t ldp, const float* decay, co
 // sequence's chunks in order; the sequence's row of state is read first and written last), every chunk's read-outs.
 // Chunks start at the first token that the step brings for a sequence.  Chunk c of sequence b is number
 // sum_{b' < b} ceil(n_b' / LC_T) + c in the scratch array, which holds H D V floats a chunk.
-#define LC_T 64        // tokens of a chunk
-#define LC_V 64        // value channels of a workgroup
-#define LC_VLD 80      // floats between two tokens' value channels in LDS
-
-typedef float lc_f32x4 __attribute__((ext_vector_type(4)));
-
-__device__ __forceinline__ int lc_chunk_base(const int* __restrict__ cu_seqlens, int b) {
-  int base = 0;
-  for (int i = 0; i < b; ++i) base += (cu_seqlens[i + 1] - cu_seqlens[i] + LC_T - 1) / LC_T;
-  return base;
-}
-
-// A chunk's rows of one projection on their way into LDS: first every load (all in flight together), then the silu and
-// the stores.  W numbers a row (WP in LDS, a multiple of 16; zeros behind W and behind the chunk's nc tokens).  VEC: rows
-// start at multiples of 16 bytes and W is a multiple of four.
-template <int WP, bool VEC>
-struct LcRows {
-  static constexpr int N = VEC ? LC_T * WP / 4 / 256 : LC_T * WP / 256;
-  float x[VEC ? 4 * N : N];
-  __device__ __forceinline__ void fetch(const float* __restrict__ src, int64_t ld, int nc, int W, int tid) {
-#pragma unroll
-    for (int i = 0; i < N; ++i) {
-      const int idx = tid + 256 * i;
-      if (VEC) {
-        const int s = idx / (WP / 4), d = 4 * (idx % (WP / 4));
-        const float4 v = s < nc && d < W ? *reinterpret_cast<const float4*>(src + (size_t)s * ld + d) : float4{0.f, 0.f, 0.f, 0.f};
-        x[4 * i] = v.x, x[4 * i + 1] = v.y, x[4 * i + 2] = v.z, x[4 * i + 3] = v.w;
-      } else {
-        const int s = idx / WP, d = idx % WP;
-        x[i] = s < nc && d < W ? src[(size_t)s * ld + d] : 0.f;
-      }
-    }
-  }
-  // dst[s * ld + d] = silu(x) * (wt ? wt[s] : 1)
-  __device__ __forceinline__ void store(float* __restrict__ dst, int ld, const float* __restrict__ wt, int tid) const {
-#pragma unroll
-    for (int i = 0; i < N; ++i) {
-      const int idx = tid + 256 * i;
-      if (VEC) {
-        const int s = idx / (WP / 4), d = 4 * (idx % (WP / 4));
-        const float w = wt ? wt[s] : 1.f;
-        *reinterpret_cast<float4*>(dst + s * ld + d) =
-            float4{w * ln_silu(x[4 * i]), w * ln_silu(x[4 * i + 1]), w * ln_silu(x[4 * i + 2]), w * ln_silu(x[4 * i + 3])};
-      } else {
-        const int s = idx / WP, d = idx % WP;
-        dst[s * ld + d] = (wt ? wt[s] : 1.f) * ln_silu(x[i]);
-      }
-    }
-  }
-};
-
 // grid (ceil(V / LC_V), H, B * NC), block 256: L_c [D][LC_V columns] = K^T (w . V), a wave to 16 value channels.
 template <int ND, bool VEC>
 __global__ __launch_bounds__(256) void lightning_chunk_state_kernel(const float* __restrict__ P, int64_t ldp,
@@ -202,9 +154,9 @@ __global__ __launch_bounds__(256) void lightning_chunk_state_kernel(const float*
   LcRows<LC_V, VEC> vr_;
   kr_.fetch(k0, ldp, nc, D, tid);
   vr_.fetch(vv0, ldp, nc, V - v0, tid);
-  kr_.store(ks, KLD, nullptr, tid);
+  kr_.store(ks, KLD, nullptr, tid, LnSilu());
   __syncthreads();
-  vr_.store(vs, LC_VLD, wt, tid);
+  vr_.store(vs, LC_VLD, wt, tid, LnSilu());
   __syncthreads();
   const int wave = tid / 64, lane = tid % 64, g = lane / 16, r = lane % 16;
   lc_f32x4 acc[ND];
@@ -295,9 +247,9 @@ __global__ __launch_bounds__(256) void lightning_chunk_out_kernel(const float* _
     qr_.fetch(q0, ldp, nc, D, tid);
     kr_.fetch(k0, ldp, nc, D, tid);
     vr_.fetch(vv0, ldp, nc, V - v0, tid);
-    qr_.store(qs, QLD, nullptr, tid);
-    kr_.store(ks, QLD, nullptr, tid);
-    vr_.store(vs, LC_VLD, nullptr, tid);
+    qr_.store(qs, QLD, nullptr, tid, LnSilu());
+    kr_.store(ks, QLD, nullptr, tid, LnSilu());
+    vr_.store(vs, LC_VLD, nullptr, tid, LnSilu());
   }
   __syncthreads();
   // scores of the wave's 16 tokens against the tokens of the column tiles up to its own

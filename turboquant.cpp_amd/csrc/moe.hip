@@ -12,8 +12,13 @@
 // router_select, one wave per token: top-k by logit, k rounds of a search in which >= lets the highest index
 // win among equal logits, so ids come out by descending logit (tq_moe.c:626-645).  Weights:
 //   renorm != 0: softmax over the selected logits (tq_moe.c:648-678);
-//   renorm == 0: softmax over all experts, the selected probabilities kept as they are.
+//   renorm == 0: softmax over all experts, the selected probabilities kept as they are;
+//   renorm == TQ_ROUTE_SIGMOID: every expert's score is the sigmoid of its logit, the choice is by score, and the weights
+//     are the selected scores over (their sum + 1e-20), times wscale.  With TQ_ROUTE_PAIR_GROUPS added, a group's score is
+//     the sum of its two largest scores.
 // shared_gate[t] = 1 / (1 + exp(-(x . shared_w)))  (tq_moe.c:1012-1018, with an exact exponential).
+#define TQ_ROUTE_SIGMOID 2
+#define TQ_ROUTE_PAIR_GROUPS 4
 #define RT 8   // most tokens per workgroup of router_logits
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
@@ -148,8 +153,10 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const float* __restr
 __device__ __forceinline__ void select_token(const float* __restrict__ src, int rows, int E, int topk, int renorm,
                                              int groups, int keep, float* lg, int* __restrict__ ids, int* ids2,
                                              float* __restrict__ weights, float* __restrict__ shared_gate,
-                                             const float* __restrict__ correction = nullptr, int n_real = 1 << 30) {
+                                             const float* __restrict__ correction = nullptr, int n_real = 1 << 30,
+                                             float wscale = 1.0f) {
   const int lane = threadIdx.x % TQ_WAVE;
+  const bool sigmoid = (renorm & TQ_ROUTE_SIGMOID) != 0, pair_groups = (renorm & TQ_ROUTE_PAIR_GROUPS) != 0;
   for (int e = lane; e < E; e += TQ_WAVE) lg[e] = src[e];
   if (rows > E && lane == 0) shared_gate[0] = 1.0f / (1.0f + expf(-src[E]));
   __builtin_amdgcn_wave_barrier();
@@ -162,6 +169,10 @@ __device__ __forceinline__ void select_token(const float* __restrict__ src, int 
     for (int e = lane; e < E; e += TQ_WAVE) d += expf(lg[e] - mx);
     denom = wave_sum(d);
   }
+  if (sigmoid) {
+    for (int e = lane; e < E; e += TQ_WAVE) lg[e] = 1.0f / (1.0f + expf(-lg[e]));
+    __builtin_amdgcn_wave_barrier();
+  }
   if (correction) {
     // the choice is by the softmax score plus a number per expert; the weights are the scores without it
     for (int e = lane; e < E; e += TQ_WAVE) lg[e] = expf(lg[e] - mx) * (1.0f / denom) + correction[e];
@@ -169,15 +180,18 @@ __device__ __forceinline__ void select_token(const float* __restrict__ src, int 
   }
   if (groups > 1 && keep < groups) {
     const int per = E / groups;
-    // a lane per group (in turns of 64): the group's largest logit
+    // a lane per group (in turns of 64): the group's largest logit, or the sum of its two largest scores
     float gmax[4];      // up to 256 groups
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int gi = lane + 64 * i;
-      float m = -INFINITY;
+      float m = -INFINITY, m2 = -INFINITY;
       if (gi < groups)
-        for (int e = gi * per; e < (gi + 1) * per; ++e) m = fmaxf(m, lg[e]);
-      gmax[i] = m;
+        for (int e = gi * per; e < (gi + 1) * per; ++e) {
+          m2 = fmaxf(m2, fminf(m, lg[e]));      // the second largest so far
+          m = fmaxf(m, lg[e]);
+        }
+      gmax[i] = pair_groups && per > 1 ? m + m2 : m;
     }
     // a group is kept if fewer than `keep` groups are better: a larger best logit, or the same and a higher index (the
     // order in which rounds of a search would take them, without the rounds: every lane looks at every group once)
@@ -241,7 +255,10 @@ __device__ __forceinline__ void select_token(const float* __restrict__ src, int 
     }
     __builtin_amdgcn_wave_barrier();
   }
-  if (renorm) {
+  if (sigmoid) {
+    const float s = wave_sum(lane < topk ? sel : 0.f);
+    if (lane < topk) weights[lane] = sel / (s + 1e-20f) * wscale;
+  } else if (renorm) {
     const float m = wave_max(lane < topk ? sel : -INFINITY);
     const float p = lane < topk ? expf(sel - m) : 0.f;
     const float s = wave_sum(p);
@@ -260,13 +277,14 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
                                                             int topk, int renorm, int groups, int keep,
                                                             int* __restrict__ ids, float* __restrict__ weights,
                                                             float* __restrict__ shared_gate, int T,
-                                                            const float* __restrict__ correction, int n_real) {
+                                                            const float* __restrict__ correction, int n_real,
+                                                            float wscale) {
   extern __shared__ float sm[];      // [4][E]
   const int wave = threadIdx.x / TQ_WAVE;
   const int t = blockIdx.x * 4 + wave;
   if (t >= T) return;
   select_token(logits + (size_t)t * rows, rows, E, topk, renorm, groups, keep, sm + wave * E, ids + (size_t)t * topk, nullptr,
-               weights + (size_t)t * topk, shared_gate + t, correction, n_real);
+               weights + (size_t)t * topk, shared_gate + t, correction, n_real, wscale);
 }
 
 static int launch_router_logits(const float* x, const void* wr, const void* shared_w, int wtype, int E,
@@ -320,7 +338,7 @@ static int groups_ok(int E, int topk, int groups, int keep) {
 // bias (null, or float [E]): added to the experts' logits before the choice.
 static int router_topk_impl(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E,
                             int topk, int renorm, int groups, int keep, int* ids, float* weights, float* shared_gate,
-                            float* logits, int T, int H, hipStream_t st, const float* correction, int n_real) {
+                            float* logits, int T, int H, hipStream_t st, const float* correction, int n_real, float wscale = 1.0f) {
   if (T <= 0) return 0;
   if (topk < 1 || topk > 64 || topk > E || E > 8192) return TQ_ERR_UNSUPPORTED;
   if (!groups_ok(E, topk, groups, keep)) return TQ_ERR_BAD_ARG;
@@ -328,7 +346,7 @@ static int router_topk_impl(const float* x, const void* wr, const void* shared_w
   if (rc) return rc;
   const int rows = E + (shared_w ? 1 : 0);
   hipLaunchKernelGGL(router_select_kernel, dim3((T + 3) / 4), dim3(256), (size_t)4 * E * sizeof(float), st, logits,
-                     rows, E, topk, renorm, groups, keep, ids, weights, shared_gate, T, correction, n_real);
+                     rows, E, topk, renorm, groups, keep, ids, weights, shared_gate, T, correction, n_real, wscale);
   TQ_LAUNCH_CHECK();
   return 0;
 }
@@ -663,7 +681,8 @@ __global__ __launch_bounds__(64 * NW) void select_align_kernel(const float* __re
                                                                int* __restrict__ pair_slot,
                                                                int* __restrict__ tile_expert,
                                                                int* __restrict__ n_tiles,
-                                                               const float* __restrict__ correction, int n_real) {
+                                                               const float* __restrict__ correction, int n_real,
+                                                               float wscale) {
   extern __shared__ int sm_i[];       // (NW + 1) * E ints for the order, NW * topk ids, NW * E floats for the choice
   int* cnt = sm_i;
   int* ids_l = cnt + (NW + 1) * E;
@@ -671,7 +690,7 @@ __global__ __launch_bounds__(64 * NW) void select_align_kernel(const float* __re
   const int wave = threadIdx.x / TQ_WAVE;
   if (wave < T)
     select_token(logits + (size_t)wave * rows, rows, E, topk, renorm, groups, keep, lg + wave * E, ids + (size_t)wave * topk,
-                 ids_l + wave * topk, weights + (size_t)wave * topk, shared_gate + wave, correction, n_real);
+                 ids_l + wave * topk, weights + (size_t)wave * topk, shared_gate + wave, correction, n_real, wscale);
   __syncthreads();
   align_pairs<NW>(ids_l, T * topk, E, topk, unit, cap, sorted_token, pair_slot, tile_expert, n_tiles, cnt, n_real);
 }
@@ -704,13 +723,13 @@ TQ_API int tq_moe_align(const int* ids, int n_pairs, int E, int topk, int unit, 
 static int route_impl(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E,
                       int topk, int renorm, int groups, int keep, int* ids, float* weights, float* shared_gate,
                       float* logits, int unit, int cap, int* sorted_token, int* pair_slot, int* tile_expert,
-                      int* n_tiles, int T, int H, hipStream_t st, const float* correction, int n_real) {
+                      int* n_tiles, int T, int H, hipStream_t st, const float* correction, int n_real, float wscale = 1.0f) {
   if (T <= 0) return 0;
   if (!groups_ok(E, topk, groups, keep)) return TQ_ERR_BAD_ARG;
   const size_t shmem = ((size_t)(AW + 1) * E + (size_t)AW * topk + (size_t)AW * E) * 4;
   if (T > AW || shmem > 64 * 1024) {
     const int rc = router_topk_impl(x, wr, shared_w, bias, wtype, E, topk, renorm, groups, keep, ids, weights,
-                                    shared_gate, logits, T, H, st, correction, n_real);
+                                    shared_gate, logits, T, H, st, correction, n_real, wscale);
     if (rc) return rc;
     // once the experts are chosen the logits are done with: the order by several workgroups keeps its table there
     const int n = T * topk;
@@ -729,7 +748,7 @@ static int route_impl(const float* x, const void* wr, const void* shared_w, cons
     const size_t shmem1 = ((size_t)2 * E + topk + E) * 4;
     hipLaunchKernelGGL(select_align_kernel<1>, dim3(1), dim3(64), shmem1, st, logits, E + (shared_w ? 1 : 0), E, topk,
                        renorm, groups, keep, ids, weights, shared_gate, T, unit, cap, sorted_token, pair_slot, tile_expert, n_tiles,
-                       correction, n_real);
+                       correction, n_real, wscale);
     TQ_LAUNCH_CHECK();
     return 0;
   }
@@ -737,7 +756,7 @@ static int route_impl(const float* x, const void* wr, const void* shared_w, cons
     (void)hipFuncSetAttribute((const void*)select_align_kernel<AW>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem);
   hipLaunchKernelGGL(select_align_kernel<AW>, dim3(1), dim3(64 * AW), shmem, st, logits, E + (shared_w ? 1 : 0), E, topk,
                      renorm, groups, keep, ids, weights, shared_gate, T, unit, cap, sorted_token, pair_slot, tile_expert, n_tiles,
-                       correction, n_real);
+                       correction, n_real, wscale);
   TQ_LAUNCH_CHECK();
   return 0;
 }
@@ -774,4 +793,23 @@ TQ_API int tq_route(const float* x, const void* wr, const void* shared_w, int wt
                     int* pair_slot, int* tile_expert, int* n_tiles, int T, int H, hipStream_t st) {
   return tq_route_grouped(x, wr, shared_w, wtype, E, topk, renorm, 1, 1, ids, weights, shared_gate, logits, unit, cap,
                           sorted_token, pair_slot, tile_expert, n_tiles, T, H, st);
+}
+
+// A router whose experts' scores are the sigmoids of their logits (bias: added to the logits first): the `topk` largest
+// scores, within the best `keep` of `groups` groups (1, 1: among all), whose score is their largest score or, with
+// pair_groups, the sum of their two largest; the weights are the chosen scores over (their sum + 1e-20), times wscale.
+TQ_API int tq_router_topk_sigmoid(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E,
+                                  int topk, int groups, int keep, int pair_groups, float wscale, int* ids, float* weights,
+                                  float* shared_gate, float* logits, int T, int H, hipStream_t st) {
+  return router_topk_impl(x, wr, shared_w, bias, wtype, E, topk, TQ_ROUTE_SIGMOID | (pair_groups ? TQ_ROUTE_PAIR_GROUPS : 0),
+                          groups, keep, ids, weights, shared_gate, logits, T, H, st, nullptr, E, wscale);
+}
+
+TQ_API int tq_route_sigmoid(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E, int topk,
+                            int groups, int keep, int pair_groups, float wscale, int* ids, float* weights, float* shared_gate,
+                            float* logits, int unit, int cap, int* sorted_token, int* pair_slot, int* tile_expert, int* n_tiles,
+                            int T, int H, hipStream_t st) {
+  return route_impl(x, wr, shared_w, bias, wtype, E, topk, TQ_ROUTE_SIGMOID | (pair_groups ? TQ_ROUTE_PAIR_GROUPS : 0), groups,
+                    keep, ids, weights, shared_gate, logits, unit, cap, sorted_token, pair_slot, tile_expert, n_tiles, T, H, st,
+                    nullptr, E, wscale);
 }

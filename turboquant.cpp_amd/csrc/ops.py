@@ -12,6 +12,7 @@ import dataclasses
 import math
 import os
 import re
+import struct
 
 import torch
 
@@ -104,6 +105,20 @@ _SIGNATURES = {
                      _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr],
     "tq_sample_topp": [_c_ptr, _c_int, _c_int, _c_f32, _c_f32, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr],
     "tq_set_pair_limit": [_c_f32],
+    "tq_add_terms_rmsnorm": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int,
+                             _c_f32, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
+    "tq_router_topk_sigmoid": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f32, _c_ptr,
+                               _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_route_sigmoid": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f32, _c_ptr, _c_ptr,
+                         _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_mm_scan": [_c_ptr, _c_i64, _c_ptr, _c_f32, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr,
+                   _c_ptr, _c_ptr],
+    "tq_mm_chunked": [_c_ptr, _c_i64, _c_ptr, _c_f32, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
+                      _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr],
+    "tq_mm_out": [_c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
+                  _c_i64, _c_i64, _c_ptr],
+    "tq_mm_decode": [_c_ptr, _c_i64, _c_ptr, _c_f32, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int,
+                     _c_f32, _c_ptr, _c_ptr],
     "tq_gate_heads": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "tq_lead_norm": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_ptr, _c_int, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
                      _c_ptr],
@@ -243,6 +258,7 @@ _KIND = {"gemm": "matmul", "gemm_mfma": "matmul", "gemm_f32": "matmul", "gemm_pa
          "router_topk": "moe", "route": "moe", "moe_align": "moe", "moe_combine": "moe",
          "delta_prep": "attn", "delta_scan": "attn", "delta_out": "attn", "delta_decode": "attn",
          "head_gemm": "matmul", "latent_norm": "attn", "gate_rows": "attn", "gate_heads": "attn",
+         "mm_scan": "attn", "mm_chunked": "attn", "mm_out": "attn", "mm_decode": "attn",
          "lightning_scan": "attn", "lightning_chunked": "attn", "lightning_out": "attn"}
 
 
@@ -382,11 +398,97 @@ class NormedDelta:
         return x[None]
 
 
+@dataclasses.dataclass
+class Terms:
+    """What several parts that ran side by side leave for the residual stream, not yet summed:
+    ``vector + sum_j weights[t, j] * y[pair_slot[t, j]] + sum_g coef_g * sum_s delta_g[s, t]``, ``parts`` being (coef, delta
+    float32 [S, T, H]) pairs, ``gathered`` a GatheredSum without a gate (or None) and ``vector`` float32 [H] or None.  The
+    next norm adds it all in the pass that normalises; ``materialize`` gives it as a float32 [1, T, H] tensor."""
+    parts: list
+    gathered: GatheredSum | None = None
+    vector: torch.Tensor | None = None
+
+    @staticmethod
+    def of(*terms, vector: torch.Tensor | None = None) -> "Terms":
+        """From (coef, what a part returned) pairs: partial sums, a GatheredSum, other Terms, or None."""
+        out = Terms([], None, vector)
+        for coef, t in terms:
+            if t is None:
+                continue
+            if isinstance(t, Terms):
+                _need(coef == 1.0 and (t.vector is None or out.vector is None), "terms", "terms within terms come unscaled, with one vector")
+                out.parts += t.parts
+                out.vector = t.vector if t.vector is not None else out.vector
+                t, dense, gate = t.gathered, None, None
+                if t is None:
+                    continue
+            elif isinstance(t, GatheredSum):
+                dense, gate = t.dense, t.gate
+                t = GatheredSum(t.y, t.pair_slot, t.weights)
+            else:
+                out.parts.append((float(coef), t))
+                continue
+            _need(coef == 1.0 and gate is None and out.gathered is None, "terms",
+                  "one sum over experts, unscaled and without a gate, goes with other terms")
+            out.gathered = t
+            if dense is not None:
+                out.parts.append((1.0, dense))
+        return out
+
+    def materialize(self, act) -> torch.Tensor:
+        ref = self.parts[0][1] if self.parts else self.gathered.y if self.gathered is not None else self.vector[None]
+        T = ref.shape[1] if self.parts else self.gathered.pair_slot.shape[0] if self.gathered is not None else 1
+        x = torch.zeros((T, ref.shape[-1]), dtype=torch.float32, device=ref.device)
+        add_rmsnorm(x, self, None, 0.0, act, want_act=False)
+        return x[None]
+
+
+def _add_terms_rmsnorm(x, terms: Terms, weight, eps: float, act, rows, want_act: bool, want_f32: bool):
+    k = "add_terms_rmsnorm"
+    T, H = x.shape
+    _need(len(terms.parts) <= 4, k, lambda: f"{len(terms.parts)} parts are beyond the 4 this kernel takes")
+    n = len(terms.parts)
+    for _, d in terms.parts:
+        _check(d, k, "a part", torch.float32)
+        _need(d.dim() == 3 and tuple(d.shape[1:]) == (T, H), k, lambda: f"a part must be [S, {T}, {H}], is {tuple(d.shape)}")
+    _need(sum(d.shape[0] for _, d in terms.parts) <= 128, k, "more partial sums than the 128 this kernel takes")
+    y = pair_slot = weights = None
+    topk = 0
+    if terms.gathered is not None:
+        y, pair_slot, weights = terms.gathered.y, terms.gathered.pair_slot, terms.gathered.weights
+        _check(y, k, "y", torch.float32)
+        _need(y.dim() == 2 and y.shape[1] == H, k, lambda: f"y must be [rows, {H}]")
+        _check(pair_slot, k, "pair_slot", torch.int32)
+        topk = pair_slot.shape[1]
+        _need(pair_slot.shape[0] == T and 1 <= topk <= 64, k, lambda: f"pair_slot must be [{T}, 1..64]")
+        _check(weights, k, "weights", torch.float32, (T, topk))
+    if terms.vector is not None:
+        _check(terms.vector, k, "vector", torch.float32, (H,))
+    R = T
+    if rows is not None:
+        _check(rows, k, "rows", torch.int32)
+        R = rows.numel()
+    if weight is not None:
+        _check(weight, k, "weight", tuple(_WTYPE), (H,))
+    else:
+        _need(rows is None, k, "without a weight all rows are summed")
+        want_act = want_f32 = False
+    out = torch.empty((R, H), dtype=ACT_DTYPES[dtype_name(act)], device=x.device) if want_act else None
+    out32 = torch.empty((R, H), dtype=torch.float32, device=x.device) if want_f32 else None
+    deltas = (ctypes.c_int64 * max(n, 1))(*[_ptr(d) for _, d in terms.parts])
+    sums = (ctypes.c_int * max(n, 1))(*[d.shape[0] for _, d in terms.parts])
+    coefs = (ctypes.c_float * max(n, 1))(*[c for c, _ in terms.parts])
+    _run("add_rmsnorm", library(act).tq_add_terms_rmsnorm(
+        _ptr(x), deltas, sums, coefs, n, T * H, _ptr(terms.vector), _ptr(y), _ptr(pair_slot), _ptr(weights), topk, _ptr(weight),
+        _WTYPE[weight.dtype] if weight is not None else 0, float(eps), _ptr(rows), R, _ptr(out), _ptr(out32), H, _stream()))
+    return out, out32
+
+
 def add_rmsnorm(x: torch.Tensor, delta, weight: torch.Tensor | None, eps: float, act,
                 rows: torch.Tensor | None = None, want_act: bool = True, want_f32: bool = False, stream: bool = False,
                 shift: tuple | None = None):
     """x += delta (in place, unless ``rows`` picks rows), where delta is None, float32 partial sums [S, T, H] added
-    one after the other, a GatheredSum, or a NormedDelta around either (then what is added is its RMS norm); returns
+    one after the other, a GatheredSum, Terms, or a NormedDelta around partial sums or a GatheredSum (then what is added is its RMS norm); returns
     rmsnorm(x) * weight as (activation-typed or None, float32 or None), one row per entry of ``rows`` (all rows if
     None).  ``weight`` None (with a NormedDelta only): the stream is summed and nothing is returned.  ``stream`` (with
     ``weight`` None, and delta None or a NormedDelta): the summed stream itself is returned in the activation type, for
@@ -399,6 +501,9 @@ def add_rmsnorm(x: torch.Tensor, delta, weight: torch.Tensor | None, eps: float,
     _need(x.dim() == 2, k, "x must be [T, H]")
     T, H = x.shape
     post = None
+    if isinstance(delta, Terms):
+        _need(not stream and shift is None, k, "the sum of several parts is normed, or only summed")
+        return _add_terms_rmsnorm(x, delta, weight, eps, act, rows, want_act, want_f32)
     if stream:
         _need(weight is None and rows is None and (delta is None or isinstance(delta, NormedDelta)), k,
               "the stream itself is returned for all rows, behind nothing or a normed part")
@@ -920,14 +1025,17 @@ def gemm_pair(first: dict, second: dict, act) -> tuple[torch.Tensor, torch.Tenso
     the same type) go out in one launch, so that the smaller one costs no launch of its own; anything else is two
     calls."""
     k = "gemm_pair"
-    keys = ("bias", "w2", "out_act", "a_rows", "tile_group", "n_tiles", "tile_rows", "gather", "partial_sums", "activation")
+    keys = ("bias", "w2", "out_act", "a_rows", "tile_group", "n_tiles", "tile_rows", "gather", "partial_sums", "activation",
+            "pair_limit")
     probs = []
     _need(not first.get("partial_sums", False), k, "only the second product may leave partial sums")
     for p in (first, second):
         full = {"bias": None, "w2": None, "out_act": False, "a_rows": None, "tile_group": None, "n_tiles": None,
-                "tile_rows": None, "gather": True, "partial_sums": False, "activation": "silu"}
+                "tile_rows": None, "gather": True, "partial_sums": False, "activation": "silu", "pair_limit": None}
         _need(set(p) <= set(full) | {"a", "w"}, k, lambda: f"unknown arguments {sorted(set(p) - set(full) - {'a', 'w'})}")
         full.update(p)
+        _need(full["pair_limit"] is None or (full["w2"] is not None and full["pair_limit"] > 0), k,
+              "a limit is for gated pairs and positive")
         probs.append(full)
     lib = library(act) if dtype_name(act) == "bfloat16" else None
     fused = lib is not None and hasattr(lib, "tq_gemm_mfma_pair")
@@ -957,8 +1065,8 @@ def gemm_pair(first: dict, second: dict, act) -> tuple[torch.Tensor, torch.Tenso
         vals = [_ptr(p["a"]), p["a"].stride(0), _ptr(p["a_rows"]), int(p["gather"]), _ptr(p["w"]), _ptr(p["w2"]), gstride,
                 _ptr(p["tile_group"]), _ptr(p["n_tiles"]), _ptr(p["bias"]),
                 _WTYPE[p["bias"].dtype] if p["bias"] is not None else 0, _ptr(out), N, int(p["out_act"]), M, N, K, tile_rows,
-                _gate_code(k, p["activation"])]
-        descs.append((ctypes.c_int64 * 19)(*[0 if v is None else int(v) for v in vals]))
+                _gate_code(k, p["activation"]), struct.unpack("<I", struct.pack("<f", p["pair_limit"] or 0.0))[0]]
+        descs.append((ctypes.c_int64 * 20)(*[0 if v is None else int(v) for v in vals]))
     _run(k, lib.tq_gemm_mfma_pair(descs[0], descs[1], splits, _stream()),
          "moe" if any(p["tile_group"] is not None for p in probs) else None)
     return outs[0], outs[1]
@@ -1075,14 +1183,14 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, lay
 
 
 # ------------------------------------------------------------------ routing
-def _expert_groups(k: str, E: int, top_k: int, groups) -> tuple[int, int]:
+def _expert_groups(k: str, E: int, top_k: int, groups, pairs: bool = False) -> tuple[int, int]:
     """(count, keep) of a choice within the best ``keep`` of ``count`` equal groups of neighbouring experts."""
     if groups is None:
         return 1, 1
     count, keep = int(groups[0]), int(groups[1])
     _need(1 <= count <= 256 and E % count == 0 and 1 <= keep <= count and top_k <= keep * (E // count), k,
           lambda: f"{count} groups of which {keep} are kept do not fit {E} experts with {top_k} per token")
-    if keep >= top_k or keep == count:
+    if keep == count or (keep >= top_k and not pairs):
         # nothing is ever left out: the best top_k experts lie in at most top_k groups, each of which has a better best
         # expert than any group without one of them, so all of these groups are among the kept
         return 1, 1
@@ -1090,15 +1198,26 @@ def _expert_groups(k: str, E: int, top_k: int, groups) -> tuple[int, int]:
 
 
 def router_topk(x32: torch.Tensor, router: torch.Tensor, shared_scale: torch.Tensor | None, top_k: int,
-                renormalize: bool, act, groups: tuple[int, int] | None = None, bias: torch.Tensor | None = None):
+                renormalize: bool, act, groups: tuple[int, int] | None = None, bias: torch.Tensor | None = None,
+                sigmoid: bool = False, weight_scale: float = 1.0, pair_groups: bool = False):
     """ids int32 [T, k], weights float32 [T, k], and sigmoid(x . shared_scale) float32 [T] (or None).
     ``groups`` (count, keep): only experts of the ``keep`` groups with the largest best score can be chosen.
-    ``bias`` float32 [E]: added to the experts' logits before the choice."""
+    ``bias`` float32 [E]: added to the experts' logits before the choice.
+    ``sigmoid``: no softmax; an expert's score is the sigmoid of its logit, and the weights are the chosen scores over (their
+    sum + 1e-20), times ``weight_scale`` (``renormalize`` true says so too).  ``pair_groups`` (with it): a group's score is the
+    sum of its two largest scores instead of its largest."""
     k = "router_topk"
     T, H, E, ids, weights, gate, logits = _router_outputs(k, x32, router, shared_scale, top_k)
-    count, keep = _expert_groups(k, E, top_k, groups)
+    count, keep = _expert_groups(k, E, top_k, groups, pair_groups)
     if bias is not None:
         _check(bias, k, "bias", torch.float32, (E,))
+    _need(sigmoid or (weight_scale == 1.0 and not pair_groups), k, "a weight scale and groups by their two best go with sigmoid scores")
+    _need(not sigmoid or renormalize, k, "sigmoid scores are renormalised over the chosen")
+    if sigmoid:
+        _run(k, library(act).tq_router_topk_sigmoid(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype],
+                                                    E, top_k, count, keep, int(pair_groups), float(weight_scale), _ptr(ids),
+                                                    _ptr(weights), _ptr(gate), _ptr(logits), T, H, _stream()))
+        return ids, weights, gate
     _run(k, library(act).tq_router_topk_biased(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E,
                                                top_k, int(bool(renormalize)), count, keep, _ptr(ids), _ptr(weights), _ptr(gate),
                                                _ptr(logits), T, H, _stream()))
@@ -1137,14 +1256,16 @@ def _align_outputs(T: int, topk: int, num_experts: int, unit: int, dev):
 
 def route(x32: torch.Tensor, router: torch.Tensor, shared_scale: torch.Tensor | None, top_k: int, renormalize: bool,
           unit: int, act, groups: tuple[int, int] | None = None, bias: torch.Tensor | None = None,
-          correction: torch.Tensor | None = None, identity: int = 0):
+          correction: torch.Tensor | None = None, identity: int = 0, sigmoid: bool = False, weight_scale: float = 1.0,
+          pair_groups: bool = False):
     """``router_topk`` followed by ``moe_align`` in one call: (ids, weights, gate, sorted_token, pair_slot,
     tile_expert, n_tiles), with the same results; a handful of tokens takes one kernel less.
 
     ``correction`` float32 [E] (with ``renormalize`` false and neither groups, bias nor shared gate): the softmax runs over
     all E rows of the router, the choice is by score + correction and the weights are the scores themselves.  ``identity`` n
     (with ``correction``): the router's last n rows are experts without matrices whose output is their input; their pairs
-    get ``pair_slot`` -1 and no rows in the order, and ``gate`` [T] is the sum of each token's weights for them."""
+    get ``pair_slot`` -1 and no rows in the order, and ``gate`` [T] is the sum of each token's weights for them.
+    ``sigmoid``, ``weight_scale``, ``pair_groups``: as for ``router_topk``."""
     k = "route"
     T, H, E, ids, weights, gate, logits = _router_outputs(k, x32, router, shared_scale, top_k)
     _need(unit in (16, 32, 64, 128, 256), k, "unit must be 16, 32, 64, 128 or 256")
@@ -1161,10 +1282,18 @@ def route(x32: torch.Tensor, router: torch.Tensor, shared_scale: torch.Tensor | 
                                              _stream()))
         return ids, weights, gate, sorted_token, pair_slot, tile_expert, n_tiles
     _need(identity == 0, k, "experts that are the identity come with a choice by corrected scores")
-    count, keep = _expert_groups(k, E, top_k, groups)
+    count, keep = _expert_groups(k, E, top_k, groups, pair_groups)
     if bias is not None:
         _check(bias, k, "bias", torch.float32, (E,))
+    _need(sigmoid or (weight_scale == 1.0 and not pair_groups), k, "a weight scale and groups by their two best go with sigmoid scores")
+    _need(not sigmoid or renormalize, k, "sigmoid scores are renormalised over the chosen")
     cap, sorted_token, pair_slot, tile_expert, n_tiles = _align_outputs(T, top_k, E, unit, x32.device)
+    if sigmoid:
+        _run(k, library(act).tq_route_sigmoid(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E,
+                                              top_k, count, keep, int(pair_groups), float(weight_scale), _ptr(ids), _ptr(weights),
+                                              _ptr(gate), _ptr(logits), unit, cap, _ptr(sorted_token), _ptr(pair_slot),
+                                              _ptr(tile_expert), _ptr(n_tiles), T, H, _stream()))
+        return ids, weights, gate, sorted_token, pair_slot, tile_expert, n_tiles
     _run(k, library(act).tq_route_biased(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E, top_k,
                                          int(bool(renormalize)), count, keep, _ptr(ids), _ptr(weights), _ptr(gate),
                                          _ptr(logits), unit, cap, _ptr(sorted_token), _ptr(pair_slot), _ptr(tile_expert),
@@ -1725,6 +1854,127 @@ def lightning_out(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps
     out = torch.empty((T, N), dtype=ACT_DTYPES[dtype_name(act)], device=o.device)
     _run(k, library(act).tq_lightning_out(_ptr(o), _ptr(gate), gate.stride(0), _ptr(weight), _WTYPE[weight.dtype], float(eps),
                                           _ptr(out), T, N, _stream()))
+    return out
+
+
+# ------------------------------------------------------------------ a matrix memory with exponential gates
+@dataclasses.dataclass(frozen=True)
+class MemoryDims:
+    """Heads, key width and value width of a matrix memory, and the cap of its gates."""
+    heads: int
+    dim: int
+    vdim: int
+    cap: float
+
+    @property
+    def projections(self) -> int:
+        """Numbers of a token's row of projections: q | k | v | gate | input gate | forget gate."""
+        return 2 * self.heads * (self.dim + self.vdim + 1)
+
+    @property
+    def m_offset(self) -> int:
+        return self.heads * (self.dim * self.vdim + self.dim)
+
+    @property
+    def state_floats(self) -> int:
+        """Floats of a sequence's row of state: S [heads][dim][vdim], n [heads][dim], m [heads], filled up to a multiple of 4."""
+        return -(-(self.m_offset + self.heads) // 4) * 4
+
+
+def _memory_args(k: str, proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.Tensor, d: MemoryDims) -> int:
+    _need(isinstance(proj, torch.Tensor) and proj.is_cuda and proj.dtype == torch.float32 and proj.dim() == 2
+          and proj.stride(1) == 1 and proj.shape[1] >= d.projections, k,
+          lambda: f"proj must be float32 [T, >= {d.projections}] on the GPU with unit stride along its rows")
+    _check(bias, k, "bias", torch.float32, (2 * d.heads,))
+    _check(state, k, "state", torch.float32)
+    _need(state.dim() == 2 and state.shape[1] == d.state_floats, k, lambda: f"state must be [slots, {d.state_floats}]")
+    B = runs["slots"].numel()
+    _check(runs["cu_seqlens"], k, "cu_seqlens", torch.int32, (B + 1,))
+    _check(runs["slots"], k, "slots", torch.int32, (B,))
+    return B
+
+
+def mm_scan(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.Tensor, dims: MemoryDims, act):
+    """The memory's recurrence over the step's runs of tokens, in order, from and into the sequences' rows of ``state``;
+    ``proj`` float32 [T, >= dims.projections] holds q | k | v | gate | raw input gate | raw forget gate, ``bias`` float32
+    [2 heads] the two gates' biases.  Returns (numerators [T, heads * vdim], denominators [T, heads], running maxima
+    [T, heads]), float32; the rows' own running maxima are for ``mm_out`` to write."""
+    k = "mm_scan"
+    B = _memory_args(k, proj, bias, runs, state, dims)
+    _need(dims.dim <= 1024, k, lambda: f"a key width of {dims.dim} is beyond the 1,024 this kernel takes")
+    T, dev = proj.shape[0], proj.device
+    num = torch.empty((T, dims.heads * dims.vdim), dtype=torch.float32, device=dev)
+    den = torch.empty((T, dims.heads), dtype=torch.float32, device=dev)
+    mrow = torch.empty((T, dims.heads), dtype=torch.float32, device=dev)
+    _run(k, library(act).tq_mm_scan(_ptr(proj), proj.stride(0), _ptr(bias), dims.cap, _ptr(runs["cu_seqlens"]), _ptr(runs["slots"]),
+                                    _ptr(state), state.stride(0), B, dims.heads, dims.dim, dims.vdim, _ptr(num), _ptr(den),
+                                    _ptr(mrow), _stream()))
+    return num, den, mrow
+
+
+def mm_chunked(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.Tensor, dims: MemoryDims, act):
+    """``mm_scan`` for steps with long runs: the same sums over chunks of 64 tokens on the matrix cores, in float32 on both
+    libraries (three launches), key widths of up to 256.  ``runs`` also names ``max_new``, the longest run.  Returns
+    (numerators, denominators); the rows of state are complete."""
+    k = "mm_chunked"
+    B = _memory_args(k, proj, bias, runs, state, dims)
+    _need(dims.dim <= 256, k, lambda: f"a key width of {dims.dim} is beyond the 256 this kernel takes")
+    T, dev, max_new = proj.shape[0], proj.device, int(runs["max_new"])
+    _need(1 <= max_new <= T, k, lambda: f"the longest run has {max_new} of {T} tokens")
+    chunks = T // LIGHTNING_CHUNK + B
+    scratch = torch.empty((chunks, dims.m_offset), dtype=torch.float32, device=dev)
+    scal = torch.empty((chunks, dims.heads, 3), dtype=torch.float64, device=dev)
+    num = torch.empty((T, dims.heads * dims.vdim), dtype=torch.float32, device=dev)
+    den = torch.empty((T, dims.heads), dtype=torch.float32, device=dev)
+    _run(k, library(act).tq_mm_chunked(_ptr(proj), proj.stride(0), _ptr(bias), dims.cap, _ptr(runs["cu_seqlens"]),
+                                       _ptr(runs["slots"]), _ptr(state), state.stride(0), B, dims.heads, dims.dim, dims.vdim,
+                                       max_new, _ptr(scratch), _ptr(scal), chunks, _ptr(num), _ptr(den), _stream()))
+    return num, den
+
+
+def mm_out(num: torch.Tensor, den: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, dims: MemoryDims, act,
+           mrow: torch.Tensor | None = None, slot_of_token: torch.Tensor | None = None, state: torch.Tensor | None = None):
+    """Every head's read-out num / den divided by its root mean square, times ``weight`` [heads * vdim] and sigmoid(gate), in the
+    activation type [T, heads * vdim].  ``mrow`` (from ``mm_scan``) with ``slot_of_token`` and ``state``: the running maxima of
+    every run's last token go into the rows of state."""
+    k = "mm_out"
+    T, N = num.shape
+    _check(num, k, "num", torch.float32, (T, dims.heads * dims.vdim))
+    _check(den, k, "den", torch.float32, (T, dims.heads))
+    _need(isinstance(gate, torch.Tensor) and gate.is_cuda and gate.dtype == torch.float32 and tuple(gate.shape) == (T, N)
+          and gate.stride(1) == 1, k, lambda: f"gate must be float32 [{T}, {N}] on the GPU with unit stride along its rows")
+    _check(weight, k, "weight", tuple(_WTYPE), (N,))
+    if mrow is not None:
+        _check(mrow, k, "mrow", torch.float32, (T, dims.heads))
+        _check(slot_of_token, k, "slot_of_token", torch.int32, (T,))
+        _check(state, k, "state", torch.float32)
+        _need(state.dim() == 2 and state.shape[1] == dims.state_floats, k, lambda: f"state must be [slots, {dims.state_floats}]")
+    out = torch.empty((T, N), dtype=ACT_DTYPES[dtype_name(act)], device=num.device)
+    _run(k, library(act).tq_mm_out(_ptr(num), _ptr(den), _ptr(gate), gate.stride(0), _ptr(weight), _WTYPE[weight.dtype], float(eps),
+                                   _ptr(out), T, dims.heads, dims.vdim, _ptr(mrow), _ptr(slot_of_token),
+                                   _ptr(state) if mrow is not None else None, state.stride(0) if mrow is not None else 0,
+                                   dims.m_offset, _stream()))
+    return out
+
+
+def mm_decode_fits(proj: torch.Tensor, dims: MemoryDims) -> bool:
+    """Whether ``mm_decode`` takes these sizes (rows that start at multiples of 16 bytes, whole groups of four channels)."""
+    return (dims.vdim % 4 == 0 and dims.vdim <= 1024 and dims.dim <= 1024 and (2 * dims.heads * dims.dim) % 4 == 0
+            and proj.stride(0) % 4 == 0 and proj.data_ptr() % 16 == 0)
+
+
+def mm_decode(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.Tensor, weight: torch.Tensor, eps: float,
+              dims: MemoryDims, act) -> torch.Tensor:
+    """``mm_scan`` and ``mm_out`` of a step of one token per sequence, in one launch."""
+    k = "mm_decode"
+    B = _memory_args(k, proj, bias, runs, state, dims)
+    _need(proj.shape[0] == B, k, "decoding brings one token per sequence")
+    N = dims.heads * dims.vdim
+    _check(weight, k, "weight", tuple(_WTYPE), (N,))
+    out = torch.empty((B, N), dtype=ACT_DTYPES[dtype_name(act)], device=proj.device)
+    _run(k, library(act).tq_mm_decode(_ptr(proj), proj.stride(0), _ptr(bias), dims.cap, _ptr(runs["slots"]), _ptr(state),
+                                      state.stride(0), B, dims.heads, dims.dim, dims.vdim, _ptr(weight), _WTYPE[weight.dtype],
+                                      float(eps), _ptr(out), _stream()))
     return out
 
 

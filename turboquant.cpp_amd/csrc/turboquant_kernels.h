@@ -51,6 +51,9 @@ int tq_gate_heads(const void* o, const float* gate, int64_t ldg, void* out, int 
 int tq_lead_norm(const float* in, int64_t ld_in, const void* w, int wtype, float eps, void* out, int out_is_act,
         int64_t ld_out, int copies, int R, int lead, int Rp, int T, hipStream_t st);
 int tq_set_pair_limit(float limit);
+int tq_add_terms_rmsnorm(float* x, const int64_t* deltas, const int* S, const float* coef, int n, int64_t delta_stride,
+        const float* vec, const float* y, const int* pair_slot, const float* weights, int topk, const void* w, int wtype,
+        float eps, const int* rows, int R, void* out, float* out32, int H, hipStream_t st);
 int tq_moe_combine(const float* y, const int* pair_slot, const float* weights, int topk, const float* shared,
         int S, int64_t shared_stride, const float* gate, float* out, int T, int H, hipStream_t st);
 int tq_embed_pos(const int* tokens, const int* positions, const void* table, const void* pos_table, int wtype, float* x,
@@ -153,6 +156,17 @@ int tq_lightning_chunked(const float* P, int64_t ldp, const float* decay, const 
         float* o, hipStream_t st);
 int tq_lightning_out(const float* o, const float* gate, int64_t ldg, const void* w, int wtype, float eps, void* out,
         int T, int N, hipStream_t st);
+// matrix_memory.hip: a matrix memory with exponential gates over a state per sequence (both libraries)
+int tq_mm_scan(const float* P, int64_t ldp, const float* bias, float cap, const int* cu_seqlens, const int* slots,
+        float* state, int64_t state_stride, int B, int H, int D, int V, float* num, float* den, float* mrow, hipStream_t st);
+int tq_mm_chunked(const float* P, int64_t ldp, const float* bias, float cap, const int* cu_seqlens, const int* slots,
+        float* state, int64_t state_stride, int B, int H, int D, int V, int max_new, float* scratch, double* scal,
+        int max_chunks, float* num, float* den, hipStream_t st);
+int tq_mm_out(const float* num, const float* den, const float* gate, int64_t ldg, const void* w, int wtype, float eps,
+        void* out, int T, int H, int V, const float* mrow, const int* slot_of_token, float* state, int64_t state_stride,
+        int64_t m_offset, hipStream_t st);
+int tq_mm_decode(const float* P, int64_t ldp, const float* bias, float cap, const int* slots, float* state,
+        int64_t state_stride, int B, int H, int D, int V, const void* w, int wtype, float eps, void* out, hipStream_t st);
 // head_gemm.hip: a product per head, out[t][h N + n] = sum_k a[t][h K + k] w[h][n][k] (both libraries)
 int tq_head_gemm(const void* a, int a_type, int64_t lda, const void* w, int wtype, void* out, int out_act, int64_t ldc,
         const float* gate, int64_t ldg, int gate_kind, int T, int H, int N, int K, hipStream_t st);
@@ -181,6 +195,13 @@ int tq_route_biased(const float* x, const void* wr, const void* shared_w, const 
 int tq_route_scored(const float* x, const void* wr, const float* correction, int wtype, int E, int n_real, int topk,
         int* ids, float* weights, float* id_gate, float* logits, int unit, int cap, int* sorted_token, int* pair_slot,
         int* tile_expert, int* n_tiles, int T, int H, hipStream_t st);
+// Scores are sigmoids of the logits; weights the chosen scores over their sum, times wscale.
+int tq_router_topk_sigmoid(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E,
+        int topk, int groups, int keep, int pair_groups, float wscale, int* ids, float* weights, float* shared_gate,
+        float* logits, int T, int H, hipStream_t st);
+int tq_route_sigmoid(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E, int topk,
+        int groups, int keep, int pair_groups, float wscale, int* ids, float* weights, float* shared_gate, float* logits,
+        int unit, int cap, int* sorted_token, int* pair_slot, int* tile_expert, int* n_tiles, int T, int H, hipStream_t st);
 // The *_sig forms of the attention entry points add what score_mod.h calls pb and keep: sigmoid weights with a bias per
 // head in the softmax's place, and first positions that stay visible whatever the window.
 int tq_attention_generic_sig(const void* q, const void* k_pool, const void* v_pool, const int* positions,

@@ -48,6 +48,9 @@ def _bind(part: Part, spec: PartSpec, path: str, out: list[Binding]) -> None:
     for name in spec.tensors:
         if name not in part.param_specs():
             raise ValueError(f"{path}: the plan gives a tensor for {name!r}, which {spec.kind} does not have")
+    for name, child in part.children().items():      # parts that are made of parts bring their specs as arguments
+        if isinstance(spec.args.get(name), PartSpec):
+            _bind(child, spec.args[name], f"{path}.{name}", out)
 
 
 class CausalLM:
@@ -76,6 +79,10 @@ class CausalLM:
         if plan.position_table is not None:
             self.bindings.append(Binding(self, "position_table", ParamSpec((plan.max_positions, H), role="table"),
                                          plan.position_table, "position_table"))
+        self.step_vectors = None       # [n, H] float32: vectors that schedule entries add to the stream
+        if plan.step_vectors is not None:
+            self.bindings.append(Binding(self, "step_vectors", ParamSpec((plan.n_step_vectors, H), role="bias"),
+                                         plan.step_vectors, "step_vectors"))
 
     # ------------------------------------------------------------ weights
     def tensor_table(self) -> dict:
@@ -89,6 +96,8 @@ class CausalLM:
         self.weight_bytes = load_bindings(self.bindings, reader, self.act, self.device, f32_matrices)
         if self.plan.lm_head is None:
             self.lm_head = self.embedding
+        if self.step_vectors is not None:
+            self.step_vectors = self.step_vectors.float().contiguous()      # they enter float arithmetic only
         for part in self.parts():
             part.prepare(self.device, self.act)
         return self
@@ -130,9 +139,13 @@ class CausalLM:
         x = ops.embed(b.tokens, self.embedding, self.act, scale=self.plan.embedding_scale, **learned)
         pending = None
         for entry, e in enumerate(self.schedule):
+            if e.step_vector is not None:      # it joins what the next norm adds into the stream
+                if isinstance(pending, ops.NormedDelta) or getattr(pending, "gate", None) is not None:
+                    pending = pending.materialize(self.act)
+                pending = ops.Terms.of((1.0, pending), vector=self.step_vectors[e.step_vector])
             pending = self.blocks[e.layer].forward(x, pending, ctx, entry)
             if ctx.layer_hook is not None:      # the stream with what the entry has left for the next norm to add
-                held = pending.materialize(self.act) if isinstance(pending, (ops.GatheredSum, ops.NormedDelta)) else pending
+                held = pending.materialize(self.act) if isinstance(pending, (ops.GatheredSum, ops.NormedDelta, ops.Terms)) else pending
                 ctx.layer_hook(entry, x.clone() if held is None else x + held.sum(0), b)
         if b.n_want == 0:
             return torch.empty((0, self.plan.vocab_size), dtype=torch.float32, device=x.device)

@@ -26,6 +26,8 @@ class NativeModel:
         self.lib = host_api.library(model.act)
         if getattr(model, "position_table", None) is not None:
             raise ValueError("the step executor embeds tokens without a learned vector per position")
+        if getattr(model, "step_vectors", None) is not None:
+            raise ValueError("the step executor adds no vectors between layers")
         if model.plan.logit_scale != 1.0:
             raise ValueError("the step executor does not multiply its logits by a constant")
         layers = [b.native() for b in model.blocks]

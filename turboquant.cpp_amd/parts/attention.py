@@ -241,6 +241,35 @@ class GroupedQueryAttention(Part):
             opts["keep_first"] = self.keep_first
         return opts
 
+    # the product of the layer's input, for an arrangement that makes it together with another mixer's (parts/parallel.py)
+    def input_weight(self) -> torch.Tensor | None:
+        """The matrix of q, k and v where nothing but the product stands between the input and the rotation, else None."""
+        if (not self.separate_qkv or self.qkv_bias is not None or self.qk_norm_eps is not None or self.rotated_norm_eps is not None
+                or self.has_head_gate or self.shares_kv or self.value_norm_eps is not None or self.value_mix is not None
+                or getattr(self.position, "amplitude", 1.0) != 1.0):
+            return None
+        return self.qkv_weight
+
+    def take_input_weight(self, weight: torch.Tensor) -> None:
+        self.qkv_weight = weight
+
+    def projects_alone(self, n_tokens: int, normed) -> bool:
+        """Whether a step of so few tokens stores its keys and values in the launch of the product (``qkv_rope_write``)."""
+        return (n_tokens <= 16 and normed.dtype == torch.bfloat16 and self.head_dim % 32 == 0 and self.hidden_size % 8 == 0
+                and self.position.rotary_dim in (0, self.head_dim) and self.position.pairing_code == 0)
+
+    def forward_projected(self, proj, ctx, entry):
+        """What follows the product of the layer's input: rotation and cache write, attention, output product."""
+        b, kv = ctx.batch, ctx.kv(entry)
+        q = ops.rope_kv_write(proj, b.positions, b.slot_of_token, kv.table, self.position.table(ctx.device),
+                              self.position.pairing_code, self.position.rotary_dim, kv.k_pages if kv.owns else None,
+                              kv.v_pages if kv.owns else None, kv.layer_offset, kv.page_size, kv.page_stride, self.num_heads,
+                              self.num_kv_heads, self.head_dim, ctx.act, runs=b.runs())
+        o = ops.attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table, kv.page_size,
+                          kv.page_stride, self.num_heads, self.num_kv_heads, self.head_dim, self.window, self.scale, ctx.act,
+                          runs=b.runs(), **self._score_options())
+        return ops.gemm(o, self.out_weight, ctx.act, bias=self.out_bias, partial_sums=True)
+
     def forward(self, normed, ctx, entry):
         b, kv = ctx.batch, ctx.kv(entry)
         amplitude = getattr(self.position, "amplitude", 1.0)

@@ -15,6 +15,8 @@ Interfaces (``ctx`` is the :class:`~..engine.context.StepContext` of the running
             state (``ctx.state(entry)``; ``ctx.state_rows(entry)`` / ``ctx.store_state_rows(entry, rows)`` read and
             write the rows of the step's sequences through the slots on the device, which a decode step that is to
             be replayed must use).  ``cache_need()`` / ``state_need()`` say what storage each run wants.
+            A mixer whose work begins with one product of its input may also offer that product to an arrangement
+            (``input_weight``, ``take_input_weight``, ``projects_alone``, ``forward_projected``; ``parts/parallel.py``).
 * ffn       ``forward(normed, normed32, ctx) -> delta``; ``wants_f32`` says whether it reads the float32 copy.
 * shift     ``forward(x, ctx, entry) -> h``: what a mixer reads of the float32 stream ``x`` where every token is blended with
             the one before it; ``state_need()`` says what it keeps per sequence between steps.
@@ -24,7 +26,8 @@ Interfaces (``ctx`` is the :class:`~..engine.context.StepContext` of the running
 
 ``delta`` is float32 [S, T, H], S partial results that the next norm adds to the stream in order, or a
 ``csrc.ops.GatheredSum``: a weighted sum over rows of a matrix (the experts' outputs) that is left to the next
-norm, whose ``materialize`` gives the tensor to an arrangement that needs it earlier.
+norm, whose ``materialize`` gives the tensor to an arrangement that needs it earlier; ``csrc.ops.Terms``: several of these
+with a factor each, from parts that ran side by side.
 """
 from __future__ import annotations
 

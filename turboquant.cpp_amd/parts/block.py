@@ -52,6 +52,35 @@ class PreNormBlock(Part):
         return self.ffn.forward(normed, normed32, ctx)
 
 
+@register_part("block", "parallel")
+class ParallelBlock(Part):
+    """One norm, whose output both halves read, and one residual sum: ``x += mixer(norm(x)) + ffn(norm(x))``, the feed-forward
+    optional.  What the halves return stays unsummed (``ops.Terms``) and is added into the stream by the next norm."""
+    graph_safe = True
+    slots = {"norm": "norm", "mixer": "mixer", "ffn": "ffn"}
+    optional = ("ffn",)
+
+    def __init__(self, norm, mixer, ffn=None):
+        self.norm, self.mixer, self.ffn = norm, mixer, ffn
+
+    def children(self):
+        parts = {"norm": self.norm, "mixer": self.mixer, "ffn": self.ffn}
+        return {k: v for k, v in parts.items() if v is not None}
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    def state_need(self):
+        return self.mixer.state_need()
+
+    def forward(self, x, pending, ctx, entry):
+        from ..csrc import ops
+        normed, normed32 = self.norm.forward(x, pending, ctx, want_f32=getattr(self.ffn, "wants_f32", False))
+        mixed = self.mixer.forward(normed, ctx, entry)
+        fed = None if self.ffn is None else self.ffn.forward(normed, normed32, ctx)
+        return ops.Terms.of((1.0, mixed), (1.0, fed))
+
+
 @register_part("block", "sandwich")
 class SandwichBlock(Part):
     """A norm before and a norm after every part: ``x += norm_b(mixer(norm_a(x))); x += norm_d(ffn(norm_c(x)))``, the

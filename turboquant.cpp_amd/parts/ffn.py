@@ -10,7 +10,10 @@ with its weight in the order chosen; the shared expert, scaled by ``sigmoid(x . 
 last.  ``renormalize`` false keeps the softmax over all experts un-normalised for the chosen ones; true is
 the reference's softmax over the chosen logits.  ``router_bias``: a number per expert is added to its logit before the
 choice.  ``pair_limit`` L: an expert is ``down(f(min(gate x, L)) * (clamp(up x, -L, L) + 1))``.  ``groups`` (count, keep): the experts form ``count`` equal groups of
-neighbours, a group's score is the largest score in it, and only experts of the ``keep`` best groups can be chosen.
+neighbours, a group's score is the largest score in it (``pair_groups``: the sum of its two largest), and only experts of
+the ``keep`` best groups can be chosen.  ``sigmoid_scores``: an expert's score is the sigmoid of its logit, the choice is by
+score, and the weights are the chosen scores over (their sum + 1e-20), times ``weight_scale``.  ``shared_limit`` L: the
+shared expert's pair is clamped as ``pair_limit`` clamps the experts' (the two may differ).
 ``gated`` false: an expert is ``down(f(up x))``, two matrices and no gate.  ``score_correction``: the softmax runs over all
 of the router's rows, the choice is by score plus a learned number per row, and the weights are the scores themselves,
 not renormalised.  ``identity`` n (with ``score_correction``): the router has n more rows than there are experts with
@@ -92,7 +95,16 @@ class SparseMoE(Part):
     def __init__(self, hidden_size: int, num_experts: int, top_k: int, expert_size: int, shared_size: int = 0,
                  shared_gated: bool = True, renormalize: bool = False, activation: str = "silu",
                  groups: tuple[int, int] | None = None, router_bias: bool = False, pair_limit: float | None = None,
-                 gated: bool = True, score_correction: bool = False, identity: int = 0):
+                 gated: bool = True, score_correction: bool = False, identity: int = 0, sigmoid_scores: bool = False,
+                 weight_scale: float = 1.0, pair_groups: bool = False, shared_limit: float | None = None):
+        if sigmoid_scores and (score_correction or not renormalize or not gated):
+            raise ValueError("sigmoid scores are renormalised over the chosen experts, which are gated pairs, and come without a correction")
+        if not sigmoid_scores and (weight_scale != 1.0 or pair_groups):
+            raise ValueError("a weight scale and groups by their two best scores go with sigmoid scores")
+        if shared_limit is not None and not (shared_size > 0 and shared_limit > 0):
+            raise ValueError(f"shared_limit is for a shared expert and positive, got {shared_limit}")
+        self.sigmoid_scores, self.weight_scale, self.pair_groups = sigmoid_scores, float(weight_scale), bool(pair_groups)
+        self.shared_limit = shared_limit
         if score_correction and (renormalize or groups is not None or router_bias or shared_size > 0):
             raise ValueError("a choice by corrected scores goes with plain softmax weights over all rows, without groups, "
                              "a router bias or a shared expert")
@@ -103,8 +115,6 @@ class SparseMoE(Part):
         self.gated, self.score_correction, self.identity, self.correction = gated, score_correction, int(identity), None
         if pair_limit is not None and not pair_limit > 0:
             raise ValueError(f"pair_limit must be positive, got {pair_limit}")
-        if (router_bias or pair_limit is not None) and shared_size > 0:
-            raise ValueError("a router with a bias and experts with a limit come without a shared expert")
         self.has_router_bias, self.pair_limit, self.router_bias = router_bias, pair_limit, None
         if not 1 <= top_k <= num_experts + identity:
             raise ValueError(f"top_k {top_k} must be within 1..{num_experts + identity}, the router's rows")
@@ -152,7 +162,8 @@ class SparseMoE(Part):
     def native(self):
         from ..csrc import host_api
         w = host_api.weight
-        if self.groups is not None or self.has_router_bias or self.pair_limit is not None or not self.gated or self.score_correction:
+        if (self.groups is not None or self.has_router_bias or self.pair_limit is not None or not self.gated or self.score_correction
+                or self.sigmoid_scores or self.shared_limit is not None):
             return None                  # the executor chooses among all experts, by logits without a bias, for plain pairs
         return host_api.MoeFfnDesc(self.hidden_size, self.num_experts, self.top_k, self.expert_size, self.shared_size,
                                    int(self.renormalize), ops.GATES[self.activation], w(self.router),
@@ -168,15 +179,18 @@ class SparseMoE(Part):
         route = lambda: ops.route(normed32, self.router, self.shared_scale if self.shared_gated else None,
                                   self.top_k, self.renormalize, unit, ctx.act,
                                   **({} if self.groups is None else {"groups": self.groups}),
-                                  **({} if self.router_bias is None else {"bias": self.router_bias}))
+                                  **({} if self.router_bias is None else {"bias": self.router_bias}),
+                                  **({} if not self.sigmoid_scores else {"sigmoid": True, "weight_scale": self.weight_scale,
+                                                                         "pair_groups": self.pair_groups}))
+        limit = {} if self.pair_limit is None else {"pair_limit": self.pair_limit}
         if self.shared_size > 0 and T <= 16 and unit == 16:
             # a handful of tokens: the shared expert's two products ride in the launches of the routed experts'
             _, weights, gate, sorted_token, pair_slot, tile_expert, n_tiles = route()
             experts = dict(a_rows=sorted_token, tile_group=tile_expert, n_tiles=n_tiles, tile_rows=unit)
             h, hs = ops.gemm_pair(dict(a=normed, w=self.expert_gate, w2=self.expert_up, out_act=True,
-                                       activation=self.activation, **experts),
+                                       activation=self.activation, **experts, **limit),
                                   dict(a=normed, w=self.shared_gate, w2=self.shared_up, out_act=True,
-                                       activation=self.activation), ctx.act)
+                                       activation=self.activation, **self._shared_limit()), ctx.act)
             y, shared = ops.gemm_pair(dict(a=h, w=self.expert_down, gather=False, **experts),
                                       dict(a=hs, w=self.shared_down, partial_sums=True), ctx.act)
             return ops.GatheredSum(y, pair_slot, weights, shared, gate)
@@ -202,8 +216,7 @@ class SparseMoE(Part):
         _, weights, gate, sorted_token, pair_slot, tile_expert, n_tiles = route()
         rows = ops.expert_product_rows(unit, T * self.top_k, self.num_experts)
         h = ops.gemm(normed, self.expert_gate, ctx.act, w2=self.expert_up, out_act=True, a_rows=sorted_token,
-                     tile_group=tile_expert, n_tiles=n_tiles, tile_rows=rows, activation=self.activation,
-                     **({} if self.pair_limit is None else {"pair_limit": self.pair_limit}))
+                     tile_group=tile_expert, n_tiles=n_tiles, tile_rows=rows, activation=self.activation, **limit)
         y = ops.gemm(h, self.expert_down, ctx.act, a_rows=sorted_token, tile_group=tile_expert, n_tiles=n_tiles,
                      tile_rows=rows, gather=False)
         if side is not None:
@@ -230,6 +243,10 @@ class SparseMoE(Part):
         # expert's output would
         return ops.GatheredSum(y, pair_slot, weights, normed32[None] if self.identity else None, own if self.identity else None)
 
+    def _shared_limit(self) -> dict:
+        return {} if self.shared_limit is None else {"pair_limit": self.shared_limit}
+
     def _shared(self, normed, ctx):
-        hs = ops.gemm(normed, self.shared_gate, ctx.act, w2=self.shared_up, out_act=True, activation=self.activation)
+        hs = ops.gemm(normed, self.shared_gate, ctx.act, w2=self.shared_up, out_act=True, activation=self.activation,
+                      **self._shared_limit())
         return ops.gemm(hs, self.shared_down, ctx.act, partial_sums=True)
