@@ -119,8 +119,9 @@ def dense_ff(h: np.ndarray, w: dict, p: str) -> np.ndarray:
     return (gelu_tanh(h @ w[p + "gate"].T) * (h @ w[p + "up"].T)) @ w[p + "down"].T
 
 
-def choose(s: np.ndarray, r: dict):
-    """scores [T, experts] -> the chosen experts [T, top] (best first) and their weights."""
+def choose(s: np.ndarray, r: dict, margins: list | None = None):
+    """scores [T, experts] -> the chosen experts [T, top] (best first) and their weights; how clear the choices were is
+    appended to ``margins``."""
     T, E = s.shape
     top, groups = r["top"], r.get("groups")
     allowed = np.ones((T, E), dtype=bool)
@@ -133,6 +134,13 @@ def choose(s: np.ndarray, r: dict):
         allowed = np.repeat(kept, per, axis=-1)
     ids = np.argsort(np.where(allowed, -s, np.inf), axis=-1, kind="stable")[:, :top]
     chosen = np.take_along_axis(s, ids, axis=-1)
+    if margins is not None:      # by how much the last chosen group and expert were ahead of the first left out
+        def ahead(scores, n):
+            order = np.sort(scores, axis=-1)[:, ::-1]
+            return order[:, n - 1] - order[:, n] if n < scores.shape[1] else np.full(T, np.inf)
+        margins.append(ahead(np.where(allowed, s, -np.inf), top))
+        if groups is not None:
+            margins.append(ahead(by_group, groups["keep"]))
     return ids, chosen / (chosen.sum(-1, keepdims=True) + 1e-20) * r["scale"]
 
 
@@ -142,8 +150,8 @@ def expert(h: np.ndarray, w: dict, p: str, limit: float) -> np.ndarray:
     return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[p + "down"].T
 
 
-def experts_ff(h: np.ndarray, f: dict, w: dict, p: str) -> np.ndarray:
-    ids, weights = choose(sigmoid(h @ w[p + "router"].T), f["router"])
+def experts_ff(h: np.ndarray, f: dict, w: dict, p: str, margins: list | None = None) -> np.ndarray:
+    ids, weights = choose(sigmoid(h @ w[p + "router"].T), f["router"], margins)
     out = np.zeros((h.shape[0], w[p + "e0.down"].shape[0]))
     for t in range(h.shape[0]):
         for e, wt in zip(ids[t], weights[t]):
@@ -164,11 +172,12 @@ def runs(cfg: dict) -> list[tuple[int, int | None]]:
     return out + [(i, None) for i in range(loop["stop"], n)]
 
 
-def forward(cfg: dict, w: dict, tokens, return_layers: bool = False):
-    """Logits [T, vocab] of a whole sequence (and the residual stream behind every layer run)."""
+def forward(cfg: dict, w: dict, tokens, return_layers: bool = False, return_margins: bool = False):
+    """Logits [T, vocab] of a whole sequence (and the residual stream behind every layer run, or per token the smallest margin
+    by which any of its choices of experts was made)."""
     eps = cfg["norm"]["eps"]
     x = w["embed"][np.asarray(tokens)] + w["pos"][:len(tokens)]
-    streams = []
+    streams, margins = [], [np.full(len(tokens), np.inf)]
     for i, step in runs(cfg):
         layer = cfg["layers"][i]
         if step is not None:
@@ -177,8 +186,10 @@ def forward(cfg: dict, w: dict, tokens, return_layers: bool = False):
         y = mixer(h, layer["mixer"], w, f"l{i}.mix.", eps)
         f = layer.get("mlp")
         if f is not None:
-            y = y + (dense_ff(h, w, f"l{i}.mlp.") if f["kind"] == "dense" else experts_ff(h, f, w, f"l{i}.mlp."))
+            y = y + (dense_ff(h, w, f"l{i}.mlp.") if f["kind"] == "dense" else experts_ff(h, f, w, f"l{i}.mlp.", margins))
         x = x + y
         streams.append(x.copy())
     logits = rms_norm(x, w["final.norm"], eps) @ w["embed"].T
+    if return_margins:
+        return logits, np.min(margins, axis=0)
     return (logits, streams) if return_layers else logits
