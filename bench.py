@@ -35,6 +35,13 @@ does it for the Bosalix design (a norm on every part's output only and a mixer i
 windowed attention over a latent with a rotated key part; attention with head norms, unit values mixed between layers,
 sigmoid weights and a window that keeps the first positions in sight; experts of two matrices chosen by corrected scores,
 some of them the identity) beside Qwen2-MoE with experts in every layer and as many weights.
+
+    python bench.py --design gokezen [--design-sizes small,medium] [--layers 8]
+
+does it for the Gokezen design (mixer and feed-forward side by side behind one norm; windowed attention beside a matrix memory
+with exponential gates; dense gated feed-forwards and clamped experts with a shared one, chosen by sigmoid scores within
+groups, in turn; a vector added before a looped pass) beside Qwen2-MoE with dense feed-forwards and experts with a shared one
+in turn.  A layer of the design has the memory's matrices over those of the layer beside it.
 """
 from __future__ import annotations
 
@@ -365,6 +372,26 @@ def bosalix_config(z: dict, layers: int, max_positions: int) -> dict:
             "embedding": {"scale": 1.0}, "layers": out}
 
 
+def gokezen_config(z: dict, layers: int, max_positions: int) -> dict:
+    """`layers` layers, dense gated feed-forwards and routed experts with a shared one in turn, each with windowed attention and a
+    matrix memory of half as many heads side by side; all but the first and the last are a loop of one pass, so that every
+    run has tensors of its own."""
+    H, G, D = z["heads"], z["kv_heads"], z["dim"]
+    mixer = {"left": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": 1024}},
+             "right": {"heads": H // 2, "dim": D, "vdim": D, "gate_cap": 15.0}, "left_scale": 1.0, "right_scale": 0.5}
+    dense = {"kind": "dense", "ff": z["dense_ff"]}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"], "limit": 7.0}, "shared": {"ff": z["ff"], "limit": 7.0},
+           "router": {"experts": z["experts"], "top": z["top"], "scale": 2.5, "groups": {"count": z["groups"], "keep": z["keep"]}}}
+    return {"architecture": "Gokezen", "vocab": z["vocab"], "width": z["width"], "max_positions": max_positions,
+            "norm": {"eps": 1e-5}, "loop": {"start": 1, "stop": layers - 1, "times": 1},
+            "layers": [{"type": "parallel", "mixer": mixer, "mlp": moe if i % 2 else dense} for i in range(layers)]}
+
+
+def qwen_mixed_shared_config_like(z: dict, layers: int, max_positions: int) -> dict:
+    """The mixed layers with a shared expert as wide as a routed one beside the routed experts."""
+    return dict(qwen_mixed_config_like(z, layers, max_positions), shared_expert_intermediate_size=z["ff"])
+
+
 def qwen_mixed_config_like(z: dict, layers: int, max_positions: int) -> dict:
     """Qwen2-MoE's layers with the dense gated feed-forward in every other layer and routed experts in the rest."""
     return dict(qwen_config_like(z, layers, max_positions), intermediate_size=z["dense_ff"],
@@ -390,7 +417,8 @@ def design_comparison(args) -> int:
     design = {"felepel": ("Felepel", felepel_config, qwen_config_like),
               "taminex": ("Taminex", taminex_config, qwen_dense_config_like),
               "beronex": ("Beronex", beronex_config, qwen_mixed_config_like),
-              "bosalix": ("Bosalix", bosalix_config, qwen_config_like)}[args.design]
+              "bosalix": ("Bosalix", bosalix_config, qwen_config_like),
+              "gokezen": ("Gokezen", gokezen_config, qwen_mixed_shared_config_like)}[args.design]
     out = {"metric": f"{design[0]} beside Qwen2-MoE at equal sizes: prompt and decode tok/s, and milliseconds by kernel",
            "unit": "tok/s", "dtype": short, "layer_runs": layers, "data": "synthetic", "sizes": {}}
 
@@ -494,7 +522,7 @@ def main() -> int:
     ap.add_argument("--seed", type=int, default=None)
     ap.add_argument("--no-workloads", action="store_true",
                     help="leave out the two workloads of unequal prompts that the default run adds under \"workloads\"")
-    ap.add_argument("--design", default=None, choices=["felepel", "taminex", "beronex", "bosalix"],
+    ap.add_argument("--design", default=None, choices=["felepel", "taminex", "beronex", "bosalix", "gokezen"],
                     help="time this design beside Qwen2-MoE at equal sizes instead of the default workload")
     ap.add_argument("--design-sizes", default="small,medium", help="of " + ", ".join(DESIGN_SIZES))
     args = ap.parse_args()

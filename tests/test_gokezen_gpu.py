@@ -726,14 +726,20 @@ def test_trace_runner_as_a_program(made, tmp_path):
                              capture_output=True, timeout=600)
         assert run.returncode == 0, run.stderr[-2000:]
         assert [l for l in run.stdout.splitlines() if l.startswith("done")] == [f"done {s['step']}" for s in steps]
-        wa, wb = plain.forward(cfg, w, a), plain.forward(cfg, w, b)
+        (wa, ca), (wb, cb) = ((plain.forward(cfg, w, t), clear_choices(cfg, w, t)) for t in (a, b))
         V = cfg["vocab"]
-        close = lambda a, b, what: check(a, b, what=what) if dtype == "float32" else None if np.median(errors(a, b)) < 0.08 else pytest.fail(what)
-        read = lambda i: np.fromfile(out / f"{i}.f32", dtype="<f4").reshape(-1, V)
-        close(read(0), wa[[0, 41, 79]], "step 0")
-        close(read(1), np.stack([wa[80], wb[40]]), "step 1")
+
+        def close(i, want, clear):
+            got = np.fromfile(out / f"{i}.f32", dtype="<f4").reshape(-1, V)
+            assert got.shape == want.shape
+            if dtype == "float32":
+                check(got, want, what=f"step {i}")
+            else:       # (single rows: where a choice of experts was close, rounding may have turned it)
+                assert (errors(got, want)[clear] < 0.15).all(), f"step {i}: {errors(got, want)}"
+        close(0, wa[[0, 41, 79]], ca[[0, 41, 79]])
+        close(1, np.stack([wa[80], wb[40]]), np.array([ca[80], cb[40]]))
         for i in range(9):
             if i % 2:
-                close(read(2 + i), wa[81 + i:82 + i], f"step {2 + i}")
+                close(2 + i, wa[81 + i:82 + i], ca[81 + i:82 + i])
             else:
                 assert not (out / f"{2 + i}.f32").exists()

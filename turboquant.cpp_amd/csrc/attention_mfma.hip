@@ -63,6 +63,7 @@ struct AttnArgs {
   ScoreMod mod;                 // what happens to a score before the softmax, and the chunks of positions (score_mod.h)
   const float* head_gate;       // null, or [T][ld_gate]: head h's output of token t is multiplied by sigmoid(head_gate[t][h])
   int64_t ld_gate;
+  int64_t ldo;                  // numbers between the rows of two tokens in out (nh * hd, or more for columns of a wider matrix)
 };
 
 // What softmax_tile needs of the score's changes for the QG groups of columns a lane holds: the plain scale, the cap and
@@ -618,7 +619,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > 16 ? 1
     if (p_q[g] < 0) continue;
     float inv = (MOD && a.mod.pb) ? 1.0f : 1.0f / l_run[g];
     if (a.head_gate) inv /= 1.0f + expf(-a.head_gate[(size_t)(t0 + p_q[g] - start) * a.ld_gate + h]);
-    bf16_t* orow = a.out + ((size_t)(t0 + p_q[g] - start) * a.nh + h) * hd;
+    bf16_t* orow = a.out + (size_t)(t0 + p_q[g] - start) * a.ldo + (size_t)h * hd;
 #pragma unroll
     for (int dt = 0; dt < VD; ++dt) {
       if (16 * dt < hd) {
@@ -751,7 +752,7 @@ __global__ __launch_bounds__(256) void attn_join_kernel(AttnArgs a) {
   __builtin_amdgcn_wave_barrier();
   float inv = a.mod.pb ? 1.0f : 1.0f / l;       // sigmoid weights are not normalised (every run's maximum is 0)
   if (a.head_gate) inv /= 1.0f + expf(-a.head_gate[(size_t)a.cu_seqlens[b] * a.ld_gate + h]);
-  bf16_t* orow = a.out + ((size_t)a.cu_seqlens[b] * a.nh + h) * a.hd;
+  bf16_t* orow = a.out + (size_t)a.cu_seqlens[b] * a.ldo + (size_t)h * a.hd;
   if (a.hd % 128 == 0) {      // a lane takes two neighbouring dimensions of its wave's 128: one pass over the runs, 8 bytes at a time
     const int d = 128 * wave + 2 * lane;
     float acc0 = 0.f, acc1 = 0.f;
@@ -825,13 +826,17 @@ TQ_API int64_t tq_attention_decode_scratch(int B, int nh, int hd, int max_end) {
 // output there, which lets a kernel leave them out.  head_gate (null: none), float [T][ld_gate]: the output of head h of
 // token t is multiplied by sigmoid(head_gate[t][h]) where it is normalised, before it is rounded.
 // pb, keep: sigmoid weights with a bias per head, and first positions that stay visible (score_mod.h; null, 0: neither).
-TQ_API int tq_attention_mfma_sig(const void* q, const void* k_pool, const void* v_pool, const int* block_table,
+// ldo: numbers between the rows of two tokens in out, a multiple of 4 (0: nh * hd).
+TQ_API int tq_attention_mfma_ld(const void* q, const void* k_pool, const void* v_pool, const int* block_table,
                                        int bt_stride, const int* cu_seqlens, const int* slots, const int* start, int page_size,
                                        int64_t page_stride, int B, int nh, int nkv, int hd, int window, float scale,
                                        float softcap, const float* r1, const float* r2, int chunk, const float* sink,
                                        void* out, float* partial, int decode, int max_new, int max_end, int value_width,
-                                       const float* head_gate, int64_t ld_gate, const float* pb, int keep, hipStream_t st) {
+                                       const float* head_gate, int64_t ld_gate, const float* pb, int keep, int64_t ldo,
+                                       hipStream_t st) {
   if (B <= 0) return 0;
+  if (ldo == 0) ldo = (int64_t)nh * hd;
+  if (ldo < (int64_t)nh * hd || ldo % 4 != 0) return TQ_ERR_BAD_ARG;
   if ((r1 == nullptr) != (r2 == nullptr) || chunk < 0 || softcap < 0.f || value_width < 0 || value_width > hd || (head_gate && ld_gate < nh)
       || keep < 0 || (pb && sink))
     return TQ_ERR_BAD_ARG;
@@ -841,7 +846,7 @@ TQ_API int tq_attention_mfma_sig(const void* q, const void* k_pool, const void* 
   if (decode && most_runs(max_end) > MAX_RUNS_LDS) return TQ_ERR_UNSUPPORTED;
   AttnArgs a{(const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_table, bt_stride, cu_seqlens, slots,
              start, page_size, page_stride, nh, nkv, hd, window, scale, (bf16_t*)out, partial,
-             most_runs(max_end), ScoreMod{softcap, r1, r2, chunk, sink, pb, keep}, head_gate, ld_gate};
+             most_runs(max_end), ScoreMod{softcap, r1, r2, chunk, sink, pb, keep}, head_gate, ld_gate, ldo};
   const int dt = hd / 16;
   // head sizes 64, 128 and 256 have kernels of their own in which nothing depends on hd at run time
   if (decode) {
@@ -876,6 +881,17 @@ TQ_API int tq_attention_mfma_sig(const void* q, const void* k_pool, const void* 
   }
   TQ_LAUNCH_CHECK();
   return 0;
+}
+
+TQ_API int tq_attention_mfma_sig(const void* q, const void* k_pool, const void* v_pool, const int* block_table,
+                                       int bt_stride, const int* cu_seqlens, const int* slots, const int* start, int page_size,
+                                       int64_t page_stride, int B, int nh, int nkv, int hd, int window, float scale,
+                                       float softcap, const float* r1, const float* r2, int chunk, const float* sink,
+                                       void* out, float* partial, int decode, int max_new, int max_end, int value_width,
+                                       const float* head_gate, int64_t ld_gate, const float* pb, int keep, hipStream_t st) {
+  return tq_attention_mfma_ld(q, k_pool, v_pool, block_table, bt_stride, cu_seqlens, slots, start, page_size, page_stride, B,
+                              nh, nkv, hd, window, scale, softcap, r1, r2, chunk, sink, out, partial, decode, max_new, max_end,
+                              value_width, head_gate, ld_gate, pb, keep, 0, st);
 }
 
 TQ_API int tq_attention_mfma_ex(const void* q, const void* k_pool, const void* v_pool, const int* block_table,

@@ -506,7 +506,7 @@ TQ_API int tq_mm_chunked(const float* P, int64_t ldp, const float* bias, float c
 template <class W>
 __global__ __launch_bounds__(256) void mm_out_kernel(const float* __restrict__ num, const float* __restrict__ den,
                                                      const float* __restrict__ gate, int64_t ldg, const W* __restrict__ w,
-                                                     float eps, act_t* __restrict__ out, int T, int H, int V,
+                                                     float eps, act_t* __restrict__ out, int64_t ldo, int T, int H, int V,
                                                      const float* __restrict__ mrow, const int* __restrict__ slot_of_token,
                                                      float* __restrict__ state_m, int64_t state_stride) {
   const int t = blockIdx.x, wave = threadIdx.x / TQ_WAVE, lane = threadIdx.x % TQ_WAVE;
@@ -522,22 +522,22 @@ __global__ __launch_bounds__(256) void mm_out_kernel(const float* __restrict__ n
     const float rs = d * (1.0f / sqrtf(ss / (float)V + eps));
     const float* g = gate + (size_t)t * ldg + (size_t)h * V;
     for (int i = lane; i < V; i += TQ_WAVE)
-      out[((size_t)t * H + h) * V + i] = from_f32<act_t>(row[i] * rs * to_f32(w[h * V + i]) * (1.0f / (1.0f + expf(-g[i]))));
+      out[(size_t)t * ldo + h * V + i] = from_f32<act_t>(row[i] * rs * to_f32(w[h * V + i]) * (1.0f / (1.0f + expf(-g[i]))));
   }
   if (mrow && (t == T - 1 || slot_of_token[t + 1] != slot_of_token[t]))
     for (int h = threadIdx.x; h < H; h += 256)
       state_m[(size_t)slot_of_token[t] * state_stride + h] = mrow[(size_t)t * H + h];
 }
 
-// state (with mrow): the rows of all slots, whose last H floats are m at offset m_offset.
+// ldo: numbers between the rows of two tokens in out.  state (with mrow): the rows of all slots, whose last H floats are m at offset m_offset.
 TQ_API int tq_mm_out(const float* num, const float* den, const float* gate, int64_t ldg, const void* w, int wtype, float eps,
-                     void* out, int T, int H, int V, const float* mrow, const int* slot_of_token, float* state,
+                     void* out, int64_t ldo, int T, int H, int V, const float* mrow, const int* slot_of_token, float* state,
                      int64_t state_stride, int64_t m_offset, hipStream_t st) {
   if (T <= 0) return 0;
-  if (H < 1 || V < 1 || ldg < (int64_t)H * V || !w || !gate || !den) return TQ_ERR_BAD_ARG;
+  if (H < 1 || V < 1 || ldg < (int64_t)H * V || ldo < (int64_t)H * V || !w || !gate || !den) return TQ_ERR_BAD_ARG;
   if (mrow && (!slot_of_token || !state || m_offset < 0 || state_stride < m_offset + H)) return TQ_ERR_BAD_ARG;
   TQ_DISPATCH_W(wtype, {
-    hipLaunchKernelGGL(mm_out_kernel<W>, dim3(T), dim3(256), 0, st, num, den, gate, ldg, (const W*)w, eps, (act_t*)out, T, H, V,
+    hipLaunchKernelGGL(mm_out_kernel<W>, dim3(T), dim3(256), 0, st, num, den, gate, ldg, (const W*)w, eps, (act_t*)out, ldo, T, H, V,
                        mrow, slot_of_token, state ? state + m_offset : state, state_stride);
   });
   TQ_LAUNCH_CHECK();
@@ -548,13 +548,54 @@ TQ_API int tq_mm_out(const float* num, const float* den, const float* gate, int6
 // One token per sequence (token b of the step is sequence b's): grid (H, B), block 1024.  Threads stand as RG groups of key
 // channels by V / 4 groups of value channels; a thread takes every RG-th key channel of its four value channels, MM_HOLD of
 // them at a time in registers.
+// A mixer beside the memory may have its queries, keys and values of the same step laid out by the same launch: one more
+// workgroup per token (blockIdx.x == H) turns nothing, takes the token's row of qkv (nh query heads, nkv key heads, nkv value
+// heads of hd numbers), puts the queries into q_out and keys and values (these transposed) into the page that holds the token's
+// position, as rope_kv_write does without a rotation.
 #define MM_HOLD 4
+struct MmKvWrite {
+  const float* qkv;             // rows ldp apart, like P's (null: nothing to write)
+  const int* positions;
+  const int* block_table;
+  int bt_stride;
+  act_t *q_out, *k_pool, *v_pool;
+  int page_size;
+  int64_t page_stride;
+  int nh, nkv, hd;
+};
+
+__device__ __forceinline__ void mm_write_kv(const MmKvWrite& k, int64_t ldp, int slot, int b) {
+  const float* row = k.qkv + (size_t)b * ldp;
+  const int pos = k.positions[b];
+  const int64_t page = k.block_table[(size_t)slot * k.bt_stride + pos / k.page_size];
+  const int r = pos % k.page_size, nq = k.nh * k.hd, nk = k.nkv * k.hd;
+  act_t* kp = k.k_pool + page * k.page_stride + (size_t)r * k.hd;
+  act_t* vp = k.v_pool + page * k.page_stride + r;
+  for (int i = threadIdx.x; i < nq + 2 * nk; i += blockDim.x) {
+    const act_t x = from_f32<act_t>(row[i]);
+    if (i < nq) {
+      k.q_out[(size_t)b * nq + i] = x;
+    } else if (i < nq + nk) {
+      const int h = (i - nq) / k.hd, d = (i - nq) % k.hd;
+      kp[(size_t)h * k.page_size * k.hd + d] = x;
+    } else {
+      const int h = (i - nq - nk) / k.hd, d = (i - nq - nk) % k.hd;
+      vp[((size_t)h * k.hd + d) * k.page_size] = x;
+    }
+  }
+}
+
 template <class W>
 __global__ __launch_bounds__(1024) void mm_decode_kernel(const float* __restrict__ P, int64_t ldp,
                                                          const float* __restrict__ bias, float cap,
                                                          const int* __restrict__ slots, float* __restrict__ state,
                                                          int64_t state_stride, int H, int D, int V,
-                                                         const W* __restrict__ w, float eps, act_t* __restrict__ out) {
+                                                         const W* __restrict__ w, float eps, act_t* __restrict__ out,
+                                                         int64_t ldo, MmKvWrite kvw) {
+  if ((int)blockIdx.x == H) {
+    mm_write_kv(kvw, ldp, slots[blockIdx.y], blockIdx.y);
+    return;
+  }
   __shared__ float qs[1024], ks[1024], red[16];
   __shared__ __align__(16) float part[4096];       // [RG][V]
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
@@ -629,27 +670,35 @@ __global__ __launch_bounds__(1024) void mm_decode_kernel(const float* __restrict
   const float ss = block_sum(o * o, red);
   if (tid < V) {
     const float g = row[(size_t)2 * H * D + (size_t)H * V + (size_t)h * V + tid];
-    out[((size_t)b * H + h) * V + tid] =
+    out[(size_t)b * ldo + h * V + tid] =
         from_f32<act_t>(o * (1.0f / sqrtf(ss / (float)V + eps)) * to_f32(w[h * V + tid]) * (1.0f / (1.0f + expf(-g))));
   }
 }
 
 // A decode step's memory in one launch: the recurrence on every sequence's row of state (m included), norm, weight and gate;
-// out [B][H V] in the activation type.  Takes value widths that are multiples of 4 up to 1,024 and key widths up to 1,024,
-// with rows of P and of the state that start at multiples of 16 bytes.
+// out [B][H V] in the activation type, rows ldo apart.  Takes value widths that are multiples of 4 up to 1,024 and key widths
+// up to 1,024, with rows of P and of the state that start at multiples of 16 bytes.  qkv (null: none), positions [B],
+// block_table [slots][bt_stride], q_out [B][nh hd], k_pool, v_pool (the layer's offset added): MmKvWrite.
 TQ_API int tq_mm_decode(const float* P, int64_t ldp, const float* bias, float cap, const int* slots, float* state,
                         int64_t state_stride, int B, int H, int D, int V, const void* w, int wtype, float eps, void* out,
+                        int64_t ldo, const float* qkv, const int* positions, const int* block_table, int bt_stride, void* q_out,
+                        void* k_pool, void* v_pool, int page_size, int64_t page_stride, int nh, int nkv, int hd,
                         hipStream_t st) {
   if (B <= 0) return 0;
   if (H < 1 || D < 1 || V < 1 || ldp < (int64_t)2 * H * (D + V + 1) || state_stride < (int64_t)H * ((int64_t)D * V + D + 1) ||
-      !(cap > 0.f) || !bias || !w)
+      !(cap > 0.f) || !bias || !w || ldo < (int64_t)H * V)
     return TQ_ERR_BAD_ARG;
-  if (V % 4 || V > 1024 || D > 1024 || H > 65535 || B > 65535 || ldp % 4 || state_stride % 4 || (2 * H * D) % 4 ||
+  if (qkv && (!positions || !block_table || bt_stride < 1 || !q_out || !k_pool || !v_pool || page_size < 1 || nh < 1 || nkv < 1 ||
+              hd < 1 || ldp < (int64_t)(nh + 2 * nkv) * hd))
+    return TQ_ERR_BAD_ARG;
+  if (V % 4 || V > 1024 || D > 1024 || H > 65534 || B > 65535 || ldp % 4 || state_stride % 4 || (2 * H * D) % 4 ||
       (uintptr_t)P % 16 || (uintptr_t)state % 16)
     return TQ_ERR_UNSUPPORTED;
+  const MmKvWrite kvw{qkv, positions, block_table, bt_stride, (act_t*)q_out, (act_t*)k_pool, (act_t*)v_pool, page_size,
+                      page_stride, nh, nkv, hd};
   TQ_DISPATCH_W(wtype, {
-    hipLaunchKernelGGL(mm_decode_kernel<W>, dim3(H, B), dim3(1024), 0, st, P, ldp, bias, cap, slots, state, state_stride, H, D,
-                       V, (const W*)w, eps, (act_t*)out);
+    hipLaunchKernelGGL(mm_decode_kernel<W>, dim3(H + (qkv ? 1 : 0), B), dim3(1024), 0, st, P, ldp, bias, cap, slots, state,
+                       state_stride, H, D, V, (const W*)w, eps, (act_t*)out, ldo, kvw);
   });
   TQ_LAUNCH_CHECK();
   return 0;

@@ -115,10 +115,11 @@ _SIGNATURES = {
                    _c_ptr, _c_ptr],
     "tq_mm_chunked": [_c_ptr, _c_i64, _c_ptr, _c_f32, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
                       _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr],
-    "tq_mm_out": [_c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
+    "tq_mm_out": [_c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
                   _c_i64, _c_i64, _c_ptr],
     "tq_mm_decode": [_c_ptr, _c_i64, _c_ptr, _c_f32, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int,
-                     _c_f32, _c_ptr, _c_ptr],
+                     _c_f32, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int,
+                     _c_int, _c_int, _c_ptr],
     "tq_gate_heads": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "tq_lead_norm": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_ptr, _c_int, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
                      _c_ptr],
@@ -162,6 +163,9 @@ _OPTIONAL = {
     "tq_attention_mfma_sig": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int,
                               _c_int, _c_int, _c_int, _c_int, _c_f32, _c_f32, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                               _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_int, _c_ptr],
+    "tq_attention_mfma_ld": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int,
+                             _c_int, _c_int, _c_int, _c_int, _c_f32, _c_f32, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
+                             _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_int, _c_i64, _c_ptr],
     "tq_attention_mfma_mod": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_int,
                               _c_int, _c_int, _c_int, _c_f32, _c_f32, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
                               _c_int, _c_int, _c_ptr],
@@ -1080,8 +1084,10 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, lay
               distance_bias: tuple[torch.Tensor, torch.Tensor] | None = None, chunk: int | None = None,
               sink: torch.Tensor | None = None, value_width: int | None = None,
               head_gate: torch.Tensor | None = None, sigmoid_bias: torch.Tensor | None = None,
-              keep_first: int = 0) -> torch.Tensor:
+              keep_first: int = 0, out: torch.Tensor | None = None) -> torch.Tensor:
     """Each token attends to its sequence's cached positions up to its own; returns [T, nh*hd].
+
+    ``out`` (bfloat16 only, see ``attention_writes_into``): where the result goes, columns of a wider matrix.
 
     ``value_width``: a head's value rows hold zeros behind their first ``value_width`` numbers (keys wider than values, both
     laid out at the keys' width); the output is zero there, and a kernel may leave those dimensions out.
@@ -1117,7 +1123,12 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, lay
     _need(head_gate is None or (isinstance(head_gate, torch.Tensor) and head_gate.is_cuda and head_gate.dtype == torch.float32
                                 and tuple(head_gate.shape) == (T, num_heads) and head_gate.stride(1) == 1), k,
           lambda: f"head_gate must be float32 [{T}, {num_heads}] on the GPU with unit stride along its rows")
-    out = torch.empty_like(q)
+    into = out is not None
+    if into:
+        _need(out.is_cuda and out.dtype == adt and tuple(out.shape) == tuple(q.shape) and out.stride(1) == 1
+              and out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0, k, "out must be columns of a matrix of the activation type, 16 bytes aligned")
+    else:
+        out = torch.empty_like(q)
     esz = k_pages.element_size()
     lib = library(act)
     cap = float(softcap or 0.0)
@@ -1148,14 +1159,15 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, lay
             _need(T == B, k, "decoding brings one token per sequence")
             partial = torch.empty((lib.tq_attention_decode_scratch(B, num_heads, head_dim, int(runs["max_end"])),),
                                   dtype=torch.float32, device=q.device)
-        plain = sigmoid_bias is None and keep_first == 0
-        _run("attention_mfma", (lib.tq_attention_mfma_ex if plain else lib.tq_attention_mfma_sig)(
+        plain = sigmoid_bias is None and keep_first == 0 and not into
+        _run("attention_mfma", (lib.tq_attention_mfma_ex if plain else lib.tq_attention_mfma_ld if into else lib.tq_attention_mfma_sig)(
             _ptr(q), k_pages.data_ptr() + layer_offset * esz, v_pages.data_ptr() + layer_offset * esz,
             _ptr(block_table), block_table.shape[1], _ptr(runs["cu_seqlens"]), _ptr(runs["slots"]), _ptr(runs["start"]),
             page_size, page_stride, B, num_heads, num_kv_heads, head_dim, int(window or 0), float(scale), *mod, _ptr(out),
             _ptr(partial), int(bool(runs["decode"])), int(runs["max_new"]), int(runs["max_end"]), int(value_width or 0),
-            _ptr(head_gate), head_gate.stride(0) if head_gate is not None else 0, *(() if plain else sig), _stream()))
+            _ptr(head_gate), head_gate.stride(0) if head_gate is not None else 0, *(() if plain else sig), *((out.stride(0),) if into else ()), _stream()))
         return out
+    _need(not into, k, "only the bfloat16 matrix-core kernels write into columns of a wider matrix")
     if (runs is not None and dtype_name(act) == "float32" and hasattr(lib, "tq_attention_f32") and head_dim % 4 == 0
             and head_dim <= 256 and page_size % 64 == 0 and page_stride % 4 == 0 and layer_offset % 4 == 0):
         B = runs["slots"].numel()
@@ -1180,6 +1192,11 @@ def attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, lay
                                          page_stride, T, num_heads, num_kv_heads, head_dim, int(window or 0),
                                          float(scale), *mod, *sig, _ptr(out), _stream()))
     return out if head_gate is None else gate_heads(out, head_gate, num_heads, "sigmoid", act)
+
+
+def attention_writes_into(act, head_dim: int, scale: float) -> bool:
+    """Whether ``attention`` takes ``out``: heads and scale that the bfloat16 matrix-core kernels run (with pages of whole tiles)."""
+    return dtype_name(act) == "bfloat16" and head_dim % 16 == 0 and head_dim <= 512 and scale > 0
 
 
 # ------------------------------------------------------------------ routing
@@ -1894,6 +1911,15 @@ def _memory_args(k: str, proj: torch.Tensor, bias: torch.Tensor, runs: dict, sta
     return B
 
 
+def _memory_rows(k: str, out: torch.Tensor | None, T: int, N: int, act, device) -> torch.Tensor:
+    adt = ACT_DTYPES[dtype_name(act)]
+    if out is None:
+        return torch.empty((T, N), dtype=adt, device=device)
+    _need(out.is_cuda and out.dtype == adt and tuple(out.shape) == (T, N) and out.stride(1) == 1 and out.stride(0) >= N, k,
+          lambda: f"out must be [{T}, {N}] of the activation type with unit stride along its rows")
+    return out
+
+
 def mm_scan(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.Tensor, dims: MemoryDims, act):
     """The memory's recurrence over the step's runs of tokens, in order, from and into the sequences' rows of ``state``;
     ``proj`` float32 [T, >= dims.projections] holds q | k | v | gate | raw input gate | raw forget gate, ``bias`` float32
@@ -1933,10 +1959,11 @@ def mm_chunked(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.
 
 
 def mm_out(num: torch.Tensor, den: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, dims: MemoryDims, act,
-           mrow: torch.Tensor | None = None, slot_of_token: torch.Tensor | None = None, state: torch.Tensor | None = None):
+           mrow: torch.Tensor | None = None, slot_of_token: torch.Tensor | None = None, state: torch.Tensor | None = None,
+           out: torch.Tensor | None = None):
     """Every head's read-out num / den divided by its root mean square, times ``weight`` [heads * vdim] and sigmoid(gate), in the
     activation type [T, heads * vdim].  ``mrow`` (from ``mm_scan``) with ``slot_of_token`` and ``state``: the running maxima of
-    every run's last token go into the rows of state."""
+    every run's last token go into the rows of state.  ``out``: where the result goes, columns of a wider matrix."""
     k = "mm_out"
     T, N = num.shape
     _check(num, k, "num", torch.float32, (T, dims.heads * dims.vdim))
@@ -1949,9 +1976,9 @@ def mm_out(num: torch.Tensor, den: torch.Tensor, gate: torch.Tensor, weight: tor
         _check(slot_of_token, k, "slot_of_token", torch.int32, (T,))
         _check(state, k, "state", torch.float32)
         _need(state.dim() == 2 and state.shape[1] == dims.state_floats, k, lambda: f"state must be [slots, {dims.state_floats}]")
-    out = torch.empty((T, N), dtype=ACT_DTYPES[dtype_name(act)], device=num.device)
+    out = _memory_rows(k, out, T, N, act, num.device)
     _run(k, library(act).tq_mm_out(_ptr(num), _ptr(den), _ptr(gate), gate.stride(0), _ptr(weight), _WTYPE[weight.dtype], float(eps),
-                                   _ptr(out), T, dims.heads, dims.vdim, _ptr(mrow), _ptr(slot_of_token),
+                                   _ptr(out), out.stride(0), T, dims.heads, dims.vdim, _ptr(mrow), _ptr(slot_of_token),
                                    _ptr(state) if mrow is not None else None, state.stride(0) if mrow is not None else 0,
                                    dims.m_offset, _stream()))
     return out
@@ -1963,18 +1990,54 @@ def mm_decode_fits(proj: torch.Tensor, dims: MemoryDims) -> bool:
             and proj.stride(0) % 4 == 0 and proj.data_ptr() % 16 == 0)
 
 
+@dataclasses.dataclass
+class KVWrite:
+    """Queries, keys and values of a decode step that a launch lays out beside its own work: ``qkv`` float32 [B, (nh + 2 nkv) *
+    hd], columns of the matrix whose other columns the launch reads; ``q`` [B, nh * hd] gets the queries, the pages get keys and
+    values as ``rope_kv_write`` writes them without a rotation."""
+    qkv: torch.Tensor
+    positions: torch.Tensor
+    block_table: torch.Tensor
+    k_pages: torch.Tensor
+    v_pages: torch.Tensor
+    layer_offset: int
+    page_size: int
+    page_stride: int
+    num_heads: int
+    num_kv_heads: int
+    head_dim: int
+    q: torch.Tensor
+
+
 def mm_decode(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.Tensor, weight: torch.Tensor, eps: float,
-              dims: MemoryDims, act) -> torch.Tensor:
-    """``mm_scan`` and ``mm_out`` of a step of one token per sequence, in one launch."""
+              dims: MemoryDims, act, out: torch.Tensor | None = None, kv_write: KVWrite | None = None) -> torch.Tensor:
+    """``mm_scan`` and ``mm_out`` of a step of one token per sequence, in one launch, which also does ``kv_write``."""
     k = "mm_decode"
     B = _memory_args(k, proj, bias, runs, state, dims)
     _need(proj.shape[0] == B, k, "decoding brings one token per sequence")
     N = dims.heads * dims.vdim
     _check(weight, k, "weight", tuple(_WTYPE), (N,))
-    out = torch.empty((B, N), dtype=ACT_DTYPES[dtype_name(act)], device=proj.device)
+    out = _memory_rows(k, out, B, N, act, proj.device)
+    extra = (None, None, None, 0, None, None, None, 0, 0, 0, 0, 0)
+    if kv_write is not None:
+        w, adt = kv_write, ACT_DTYPES[dtype_name(act)]
+        width = (w.num_heads + 2 * w.num_kv_heads) * w.head_dim
+        _need(w.qkv.is_cuda and w.qkv.dtype == torch.float32 and tuple(w.qkv.shape) == (B, width) and w.qkv.stride(1) == 1
+              and w.qkv.stride(0) == proj.stride(0), k, lambda: f"qkv must be float32 [{B}, {width}], columns of proj's matrix")
+        _check(w.positions, k, "positions", torch.int32, (B,))
+        _check(w.block_table, k, "block_table", torch.int32)
+        _check(w.k_pages, k, "k_pages", adt)
+        _check(w.v_pages, k, "v_pages", adt)
+        _check(w.q, k, "q", adt, (B, w.num_heads * w.head_dim))
+        _need(w.block_table.dim() == 2 and w.layer_offset + w.num_kv_heads * w.page_size * w.head_dim <= w.page_stride, k,
+              "layer does not fit in a page")
+        esz = w.k_pages.element_size()
+        extra = (_ptr(w.qkv), _ptr(w.positions), _ptr(w.block_table), w.block_table.shape[1], _ptr(w.q),
+                 w.k_pages.data_ptr() + w.layer_offset * esz, w.v_pages.data_ptr() + w.layer_offset * esz, w.page_size,
+                 w.page_stride, w.num_heads, w.num_kv_heads, w.head_dim)
     _run(k, library(act).tq_mm_decode(_ptr(proj), proj.stride(0), _ptr(bias), dims.cap, _ptr(runs["slots"]), _ptr(state),
                                       state.stride(0), B, dims.heads, dims.dim, dims.vdim, _ptr(weight), _WTYPE[weight.dtype],
-                                      float(eps), _ptr(out), _stream()))
+                                      float(eps), _ptr(out), out.stride(0), *extra, _stream()))
     return out
 
 

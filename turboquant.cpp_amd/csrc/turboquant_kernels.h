@@ -163,10 +163,12 @@ int tq_mm_chunked(const float* P, int64_t ldp, const float* bias, float cap, con
         float* state, int64_t state_stride, int B, int H, int D, int V, int max_new, float* scratch, double* scal,
         int max_chunks, float* num, float* den, hipStream_t st);
 int tq_mm_out(const float* num, const float* den, const float* gate, int64_t ldg, const void* w, int wtype, float eps,
-        void* out, int T, int H, int V, const float* mrow, const int* slot_of_token, float* state, int64_t state_stride,
-        int64_t m_offset, hipStream_t st);
+        void* out, int64_t ldo, int T, int H, int V, const float* mrow, const int* slot_of_token, float* state,
+        int64_t state_stride, int64_t m_offset, hipStream_t st);
 int tq_mm_decode(const float* P, int64_t ldp, const float* bias, float cap, const int* slots, float* state,
-        int64_t state_stride, int B, int H, int D, int V, const void* w, int wtype, float eps, void* out, hipStream_t st);
+        int64_t state_stride, int B, int H, int D, int V, const void* w, int wtype, float eps, void* out, int64_t ldo,
+        const float* qkv, const int* positions, const int* block_table, int bt_stride, void* q_out, void* k_pool,
+        void* v_pool, int page_size, int64_t page_stride, int nh, int nkv, int hd, hipStream_t st);
 // head_gemm.hip: a product per head, out[t][h N + n] = sum_k a[t][h K + k] w[h][n][k] (both libraries)
 int tq_head_gemm(const void* a, int a_type, int64_t lda, const void* w, int wtype, void* out, int out_act, int64_t ldc,
         const float* gate, int64_t ldg, int gate_kind, int T, int H, int N, int K, hipStream_t st);
@@ -213,6 +215,12 @@ int tq_attention_mfma_sig(const void* q, const void* k_pool, const void* v_pool,
         int nh, int nkv, int hd, int window, float scale, float softcap, const float* r1, const float* r2, int chunk,
         const float* sink, void* out, float* partial, int decode, int max_new, int max_end, int value_width,
         const float* head_gate, int64_t ld_gate, const float* pb, int keep, hipStream_t st);
+// the same with ldo numbers between the rows of two tokens in out
+int tq_attention_mfma_ld(const void* q, const void* k_pool, const void* v_pool, const int* block_table, int bt_stride,
+        const int* cu_seqlens, const int* slots, const int* start, int page_size, int64_t page_stride, int B,
+        int nh, int nkv, int hd, int window, float scale, float softcap, const float* r1, const float* r2, int chunk,
+        const float* sink, void* out, float* partial, int decode, int max_new, int max_end, int value_width,
+        const float* head_gate, int64_t ld_gate, const float* pb, int keep, int64_t ldo, hipStream_t st);
 int tq_attention_f32_sig(const void* q, const void* k_pool, const void* v_pool, const int* block_table, int bt_stride,
         const int* cu_seqlens, const int* slots, const int* start, int page_size, int64_t page_stride, int B,
         int nh, int nkv, int hd, int window, float scale, float softcap, const float* r1, const float* r2, int chunk,

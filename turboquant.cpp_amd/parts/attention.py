@@ -253,22 +253,35 @@ class GroupedQueryAttention(Part):
     def take_input_weight(self, weight: torch.Tensor) -> None:
         self.qkv_weight = weight
 
-    def projects_alone(self, n_tokens: int, normed) -> bool:
-        """Whether a step of so few tokens stores its keys and values in the launch of the product (``qkv_rope_write``)."""
-        return (n_tokens <= 16 and normed.dtype == torch.bfloat16 and self.head_dim % 32 == 0 and self.hidden_size % 8 == 0
-                and self.position.rotary_dim in (0, self.head_dim) and self.position.pairing_code == 0)
+    def output_weight(self) -> torch.Tensor | None:
+        return None if self.out_bias is not None else self.out_weight
 
-    def forward_projected(self, proj, ctx, entry):
-        """What follows the product of the layer's input: rotation and cache write, attention, output product."""
+    def writes_into(self, act: str) -> bool:
+        """Whether ``read_out`` can put its rows into columns of a wider matrix."""
+        return ops.attention_writes_into(act, self.head_dim, self.scale)
+
+    def kv_write(self, proj, ctx, entry) -> ops.KVWrite | None:
+        """A decode step's queries, keys and values for another launch to lay out (``read_out`` then takes the queries), or None
+        where more than that stands between the product and the cache."""
         b, kv = ctx.batch, ctx.kv(entry)
-        q = ops.rope_kv_write(proj, b.positions, b.slot_of_token, kv.table, self.position.table(ctx.device),
-                              self.position.pairing_code, self.position.rotary_dim, kv.k_pages if kv.owns else None,
-                              kv.v_pages if kv.owns else None, kv.layer_offset, kv.page_size, kv.page_stride, self.num_heads,
-                              self.num_kv_heads, self.head_dim, ctx.act, runs=b.runs())
-        o = ops.attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table, kv.page_size,
-                          kv.page_stride, self.num_heads, self.num_kv_heads, self.head_dim, self.window, self.scale, ctx.act,
-                          runs=b.runs(), **self._score_options())
-        return ops.gemm(o, self.out_weight, ctx.act, bias=self.out_bias, partial_sums=True)
+        if not b.is_decode or not kv.owns or self.position.rotary_dim != 0:
+            return None
+        q = torch.empty((proj.shape[0], self.q_size), dtype=kv.k_pages.dtype, device=proj.device)
+        return ops.KVWrite(proj, b.positions, kv.table, kv.k_pages, kv.v_pages, kv.layer_offset, kv.page_size, kv.page_stride,
+                           self.num_heads, self.num_kv_heads, self.head_dim, q)
+
+    def read_out(self, proj, ctx, entry, out=None, q=None):
+        """What follows the product of the layer's input, up to the output product: rotation and cache write (done already where
+        ``q`` gives the queries) and attention."""
+        b, kv = ctx.batch, ctx.kv(entry)
+        if q is None:
+            q = ops.rope_kv_write(proj, b.positions, b.slot_of_token, kv.table, self.position.table(ctx.device),
+                                  self.position.pairing_code, self.position.rotary_dim, kv.k_pages if kv.owns else None,
+                                  kv.v_pages if kv.owns else None, kv.layer_offset, kv.page_size, kv.page_stride, self.num_heads,
+                                  self.num_kv_heads, self.head_dim, ctx.act, runs=b.runs())
+        return ops.attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table, kv.page_size,
+                             kv.page_stride, self.num_heads, self.num_kv_heads, self.head_dim, self.window, self.scale, ctx.act,
+                             runs=b.runs(), **({} if out is None else {"out": out}), **self._score_options())
 
     def forward(self, normed, ctx, entry):
         b, kv = ctx.batch, ctx.kv(entry)

@@ -15,8 +15,8 @@ Interfaces (``ctx`` is the :class:`~..engine.context.StepContext` of the running
             state (``ctx.state(entry)``; ``ctx.state_rows(entry)`` / ``ctx.store_state_rows(entry, rows)`` read and
             write the rows of the step's sequences through the slots on the device, which a decode step that is to
             be replayed must use).  ``cache_need()`` / ``state_need()`` say what storage each run wants.
-            A mixer whose work begins with one product of its input may also offer that product to an arrangement
-            (``input_weight``, ``take_input_weight``, ``projects_alone``, ``forward_projected``; ``parts/parallel.py``).
+            A mixer that is a product of its input, something behind it and an output product may also offer these one by
+            one to an arrangement (``input_weight``, ``read_out``, ``output_weight`` and others; ``parts/parallel.py``).
 * ffn       ``forward(normed, normed32, ctx) -> delta``; ``wants_f32`` says whether it reads the float32 copy.
 * shift     ``forward(x, ctx, entry) -> h``: what a mixer reads of the float32 stream ``x`` where every token is blended with
             the one before it; ``state_need()`` says what it keeps per sequence between steps.

@@ -73,25 +73,35 @@ class MatrixMemory(Part):
     def take_input_weight(self, weight: torch.Tensor) -> None:
         self.in_weight = weight
 
-    def projects_alone(self, n_tokens: int, normed) -> bool:
-        return False
+    def output_weight(self) -> torch.Tensor:
+        return self.out_weight
 
-    def forward(self, normed, ctx, entry):
-        return self.forward_projected(ops.gemm(normed, self.in_weight, ctx.act), ctx, entry)
+    def writes_into(self, act: str) -> bool:
+        return True
 
-    def forward_projected(self, proj, ctx, entry):
+    def scale_output(self, factor: float) -> None:
+        """Multiplies what the mixer puts out: a factor on the weights of its last norm, in float32."""
+        self.out_norm = (self.out_norm.float() * factor).contiguous()
+
+    def takes_kv_write(self, proj, ctx) -> bool:
+        """Whether this step's ``read_out`` can lay out another mixer's keys and values in its launch."""
+        return ctx.batch.is_decode and ops.mm_decode_fits(proj, self.dims)
+
+    def read_out(self, proj, ctx, entry, out=None, kv_write=None):
+        """What follows the product of the layer's input, up to the output product: activation rows [T, heads * vdim]."""
         d, b, state = self.dims, ctx.batch, ctx.state(entry)
         runs = b.runs()
         if runs["decode"] and ops.mm_decode_fits(proj, d):
-            out = ops.mm_decode(proj, self.gate_bias, runs, state, self.out_norm, self.eps, d, ctx.act)
-        else:
-            at = 2 * d.heads * d.dim + d.heads * d.vdim
-            gate = proj[:, at:at + d.heads * d.vdim]
-            if runs["max_new"] >= self.chunked_from and d.dim <= 256:
-                num, den = ops.mm_chunked(proj, self.gate_bias, runs, state, d, ctx.act)
-                out = ops.mm_out(num, den, gate, self.out_norm, self.eps, d, ctx.act)
-            else:
-                num, den, mrow = ops.mm_scan(proj, self.gate_bias, runs, state, d, ctx.act)
-                out = ops.mm_out(num, den, gate, self.out_norm, self.eps, d, ctx.act, mrow=mrow, slot_of_token=b.slot_of_token,
-                                 state=state)
+            return ops.mm_decode(proj, self.gate_bias, runs, state, self.out_norm, self.eps, d, ctx.act, out=out, kv_write=kv_write)
+        at = 2 * d.heads * d.dim + d.heads * d.vdim
+        gate = proj[:, at:at + d.heads * d.vdim]
+        if runs["max_new"] >= self.chunked_from and d.dim <= 256:
+            num, den = ops.mm_chunked(proj, self.gate_bias, runs, state, d, ctx.act)
+            return ops.mm_out(num, den, gate, self.out_norm, self.eps, d, ctx.act, out=out)
+        num, den, mrow = ops.mm_scan(proj, self.gate_bias, runs, state, d, ctx.act)
+        return ops.mm_out(num, den, gate, self.out_norm, self.eps, d, ctx.act, mrow=mrow, slot_of_token=b.slot_of_token,
+                          state=state, out=out)
+
+    def forward(self, normed, ctx, entry):
+        out = self.read_out(ops.gemm(normed, self.in_weight, ctx.act), ctx, entry)
         return ops.gemm(out, self.out_weight, ctx.act, partial_sums=True)
