@@ -54,4 +54,18 @@ struct LcRows {
       }
     }
   }
+  // dst[s * WP + (d ^ 16 (s % 4))] = x, WP a multiple of 64: rows without padding whose 16 columns by 4 rows lie on 64 banks
+  __device__ __forceinline__ void store_turned(float* __restrict__ dst, int tid) const {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int idx = tid + 256 * i;
+      if (VEC) {
+        const int s = idx / (WP / 4), d = 4 * (idx % (WP / 4));
+        *reinterpret_cast<float4*>(dst + s * WP + (d ^ (16 * (s & 3)))) = float4{x[4 * i], x[4 * i + 1], x[4 * i + 2], x[4 * i + 3]};
+      } else {
+        const int s = idx / WP, d = idx % WP;
+        dst[s * WP + (d ^ (16 * (s & 3)))] = x[i];
+      }
+    }
+  }
 };

@@ -268,7 +268,7 @@ __global__ __launch_bounds__(256) void mm_chunk_state_kernel(const float* __rest
 
 // grid (ceil((D V + D) / 256), H, B), block 256: every chunk's own sums become the state before it, in place; the row of
 // state (S and n) is advanced, its m is only read.
-#define MM_AHEAD 8        // chunks whose sums are asked for before the first of them is replaced
+#define MM_AHEAD 16       // chunks whose sums are asked for before the first of them is replaced
 __global__ __launch_bounds__(256) void mm_chunk_prefix_kernel(const int* __restrict__ cu_seqlens, const int* __restrict__ slots,
                                                               float* __restrict__ state, int64_t state_stride, int max_chunks,
                                                               int H, int D, int V, float* __restrict__ scratch,
@@ -313,8 +313,10 @@ __global__ __launch_bounds__(256) void mm_chunk_prefix_kernel(const int* __restr
 
 // grid (ceil(V / LC_V), H, B * NC), block 256: a chunk's numerators for LC_V value channels, a wave to 16 tokens; the first
 // block of value channels also the denominators, and in a run's last chunk the sequence's new m.
+// (the values wait in registers until the keys have been read and take their place in LDS: with key widths of up to 128 two
+// workgroups fit a compute unit)
 template <int ND, bool VEC>
-__global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restrict__ P, int64_t ldp,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND > 8 ? 1 : 2))) void mm_chunk_out_kernel(const float* __restrict__ P, int64_t ldp,
                                                            const float* __restrict__ bias, float cap,
                                                            const int* __restrict__ cu_seqlens, const int* __restrict__ slots,
                                                            float* __restrict__ state, int64_t state_stride, int NC,
@@ -322,14 +324,14 @@ __global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restri
                                                            const float* __restrict__ scratch, const double* __restrict__ scal,
                                                            float* __restrict__ num, float* __restrict__ den) {
   extern __shared__ __align__(16) float mm_lds[];
-  constexpr int DP = 16 * ND, QLD = DP + 4, PLD = LC_T + 4, KROWS = QLD > PLD ? QLD : PLD;
+  constexpr int DP = 16 * ND, QLD = DP + 4, PLD = LC_T + 4;
   double* as = reinterpret_cast<double*>(mm_lds);      // [LC_T] a_s
   double* Ms = as + LC_T;                // [LC_T] M_t
   float* coef = reinterpret_cast<float*>(Ms + LC_T);   // [LC_T] e^(m - M_t)
   float* mt = coef + LC_T;               // [LC_T] the running maximum at t
   float* qs = mt + LC_T;                 // [LC_T][QLD]
   float* ks = qs + LC_T * QLD;           // [LC_T][QLD]; later the weighted scores [LC_T][PLD]
-  float* vs = ks + LC_T * KROWS;         // [LC_T][LC_VLD]
+  float* vs = ks + LC_T * PLD;           // and the values [LC_T][LC_V] behind them
   const int b = blockIdx.z / NC, c = blockIdx.z % NC, h = blockIdx.y, v0 = blockIdx.x * LC_V;
   const int t0 = cu_seqlens[b], n = cu_seqlens[b + 1] - t0;
   if (c * LC_T >= n) return;
@@ -339,7 +341,7 @@ __global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restri
   const int wave = tid / 64, lane = tid % 64, g = lane / 16, r = lane % 16;
   const float* chunk = scratch + (size_t)gi * H * (D * V + D);
   // the state before the chunk, as the last product's operand: asked for first, so that it arrives while the rest is staged
-  constexpr int AHEAD = DP / 4 > 32 ? 32 : DP / 4;
+  constexpr int AHEAD = DP / 4 > 16 ? 16 : DP / 4;
   const float* sb = chunk + (size_t)h * D * V + v0 + r;
   float sv[AHEAD][4];
 #pragma unroll
@@ -348,9 +350,9 @@ __global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restri
     for (int cv = 0; cv < 4; ++cv)
       sv[k4][cv] = 4 * k4 + g < D && v0 + 16 * cv + r < V ? sb[(size_t)(4 * k4 + g) * V + 16 * cv] : 0.f;
   const float* row0 = P + (size_t)(t0 + c * LC_T) * ldp;
+  LcRows<LC_V, VEC> vr_;
   {
     LcRows<DP, VEC> qr_, kr_;
-    LcRows<LC_V, VEC> vr_;
     qr_.fetch(row0 + (size_t)h * D, ldp, nc, D, tid);
     kr_.fetch(row0 + (size_t)H * D + (size_t)h * D, ldp, nc, D, tid);
     vr_.fetch(row0 + (size_t)2 * H * D + (size_t)h * V + v0, ldp, nc, V - v0, tid);
@@ -369,7 +371,6 @@ __global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restri
     }
     qr_.store(qs, QLD, nullptr, tid, MmScaled{1.0f / sqrtf((float)D)});
     kr_.store(ks, QLD, nullptr, tid, MmScaled{1.f});
-    vr_.store(vs, LC_VLD, nullptr, tid, MmScaled{1.f});
   }
   __syncthreads();
   // scores of the wave's 16 tokens against the tokens of the column tiles up to its own
@@ -384,8 +385,9 @@ __global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restri
     for (int ct = 0; ct < 4; ++ct)
       if (ct <= wave) sc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, ks[(16 * ct + r) * QLD + 4 * k4 + g], sc[ct], 0, 0, 0);
   }
-  __syncthreads();                        // every wave has read the keys: their place takes the weighted scores
+  __syncthreads();                        // every wave has read the keys: their place takes the weighted scores and the values
   float* ps = ks;
+  vr_.store_turned(vs, tid);
 #pragma unroll
   for (int ct = 0; ct < 4; ++ct)
 #pragma unroll
@@ -400,9 +402,9 @@ __global__ __launch_bounds__(256) void mm_chunk_out_kernel(const float* __restri
   const float* prow = ps + (16 * wave + r) * PLD + g;
   for (int k4 = 0; k4 < 4 * (wave + 1); ++k4) {
     const float a = prow[4 * k4];
-    const float* vr = vs + (4 * k4 + g) * LC_VLD + r;
+    const float* vr = vs + (4 * k4 + g) * LC_V + r;
 #pragma unroll
-    for (int cv = 0; cv < 4; ++cv) acc[cv] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vr[16 * cv], acc[cv], 0, 0, 0);
+    for (int cv = 0; cv < 4; ++cv) acc[cv] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vr[16 * (cv ^ g)], acc[cv], 0, 0, 0);
   }
   // what the state before the chunk adds: q S, each row times e^(m - M_t)
 #pragma unroll
@@ -452,9 +454,10 @@ template <int ND, bool VEC>
 static int mm_chunked_launch(const float* P, int64_t ldp, const float* bias, float cap, const int* cu_seqlens, const int* slots,
                              float* state, int64_t state_stride, int B, int NC, int max_chunks, int H, int D, int V,
                              float* scratch, double* scal, float* num, float* den, hipStream_t st) {
-  constexpr int DP = 16 * ND, KLD = DP + (80 - DP % 64) % 64, QLD = DP + 4, KROWS = QLD > LC_T + 4 ? QLD : LC_T + 4;
+  constexpr int DP = 16 * ND, KLD = DP + (80 - DP % 64) % 64, QLD = DP + 4,
+                KROWS = QLD > LC_T + 4 + LC_V ? QLD : LC_T + 4 + LC_V;
   const size_t sh_state = ((size_t)LC_T * KLD + (size_t)LC_T * LC_VLD + LC_T) * sizeof(float);
-  const size_t sh_out = ((size_t)LC_T * QLD + (size_t)LC_T * KROWS + (size_t)LC_T * LC_VLD + 6 * LC_T) * sizeof(float);
+  const size_t sh_out = ((size_t)LC_T * QLD + (size_t)LC_T * KROWS + 6 * LC_T) * sizeof(float);
   if (sh_state > 48 * 1024)
     (void)hipFuncSetAttribute((const void*)mm_chunk_state_kernel<ND, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize,
                               (int)sh_state);
