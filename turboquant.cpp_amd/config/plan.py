@@ -76,6 +76,9 @@ class ModelPlan:
     logit_scale: float = 1.0                # the logits are multiplied by it, before the cap
     position_table: Source | None = None    # a learned vector per position [max_positions, H], added to the embedded token
 
+    token_table: Source | None = None       # a second table with a row per token [V, token_table_width], for "side" parts
+    token_table_width: int = 0
+
     step_vectors: Source | None = None      # a vector per pass of a loop [n_step_vectors, H]: see ScheduleEntry.step_vector
     n_step_vectors: int = 0
 

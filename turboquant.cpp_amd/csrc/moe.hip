@@ -11,7 +11,7 @@
 // there are few tokens, so that decoding does not leave the chip to eight waves.
 // router_select, one wave per token: top-k by logit, k rounds of a search in which >= lets the highest index
 // win among equal logits, so ids come out by descending logit (tq_moe.c:626-645).  Weights:
-//   renorm != 0: softmax over the selected logits (tq_moe.c:648-678);
+//   renorm != 0: softmax over the selected logits (tq_moe.c:648-678), times wscale;
 //   renorm == 0: softmax over all experts, the selected probabilities kept as they are;
 //   renorm == TQ_ROUTE_SIGMOID: every expert's score is the sigmoid of its logit, the choice is by score, and the weights
 //     are the selected scores over (their sum + 1e-20), times wscale.  With TQ_ROUTE_PAIR_GROUPS added, a group's score is
@@ -262,7 +262,7 @@ __device__ __forceinline__ void select_token(const float* __restrict__ src, int 
     const float m = wave_max(lane < topk ? sel : -INFINITY);
     const float p = lane < topk ? expf(sel - m) : 0.f;
     const float s = wave_sum(p);
-    if (lane < topk) weights[lane] = s > 0.f ? p * (1.0f / s) : 0.f;
+    if (lane < topk) weights[lane] = (s > 0.f ? p * (1.0f / s) : 0.f) * wscale;
   } else {
     const float wgt = lane < topk ? expf(sel - mx) * (1.0f / denom) : 0.f;
     if (lane < topk) weights[lane] = wgt;
@@ -812,4 +812,20 @@ TQ_API int tq_route_sigmoid(const float* x, const void* wr, const void* shared_w
   return route_impl(x, wr, shared_w, bias, wtype, E, topk, TQ_ROUTE_SIGMOID | (pair_groups ? TQ_ROUTE_PAIR_GROUPS : 0), groups,
                     keep, ids, weights, shared_gate, logits, unit, cap, sorted_token, pair_slot, tile_expert, n_tiles, T, H, st,
                     nullptr, E, wscale);
+}
+
+// A router whose weights are the softmax over the chosen experts' logits, times wscale (bias: added to the logits first).
+TQ_API int tq_router_topk_weighted(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E,
+                                   int topk, int groups, int keep, float wscale, int* ids, float* weights, float* shared_gate,
+                                   float* logits, int T, int H, hipStream_t st) {
+  return router_topk_impl(x, wr, shared_w, bias, wtype, E, topk, 1, groups, keep, ids, weights, shared_gate, logits, T, H, st,
+                          nullptr, E, wscale);
+}
+
+TQ_API int tq_route_weighted(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E, int topk,
+                             int groups, int keep, float wscale, int* ids, float* weights, float* shared_gate, float* logits,
+                             int unit, int cap, int* sorted_token, int* pair_slot, int* tile_expert, int* n_tiles, int T, int H,
+                             hipStream_t st) {
+  return route_impl(x, wr, shared_w, bias, wtype, E, topk, 1, groups, keep, ids, weights, shared_gate, logits, unit, cap,
+                    sorted_token, pair_slot, tile_expert, n_tiles, T, H, st, nullptr, E, wscale);
 }

@@ -120,6 +120,30 @@ _SIGNATURES = {
     "tq_mm_decode": [_c_ptr, _c_i64, _c_ptr, _c_f32, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int,
                      _c_f32, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int,
                      _c_int, _c_int, _c_ptr],
+    "tq_router_topk_weighted": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f32, _c_ptr, _c_ptr,
+                                _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_route_weighted": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f32, _c_ptr, _c_ptr, _c_ptr,
+                          _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_add_norm": [_c_ptr, _c_ptr, _c_int, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_f32,
+                    _c_int, _c_ptr, _c_ptr, _c_f32, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
+    "tq_token_gate": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_row_norm_kv_write": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_f32, _c_ptr, _c_ptr,
+                             _c_int, _c_f32, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_int,
+                             _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_diff_prep_kv_write": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_f32, _c_int, _c_f32,
+                              _c_f32, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                              _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_diff_combine": [_c_ptr, _c_f32, _c_f32, _c_int, _c_f32, _c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
+    "tq_ssd_prep": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int,
+                    _c_ptr, _c_ptr, _c_int, _c_ptr],
+    "tq_ssd_scan": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
+                    _c_int, _c_ptr, _c_ptr],
+    "tq_ssd_chunked": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
+                       _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr],
+    "tq_ssd_decode": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
+                      _c_int, _c_int, _c_int, _c_ptr, _c_ptr],
+    "tq_ssd_out": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int,
+                   _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr],
     "tq_gate_heads": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "tq_lead_norm": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_f32, _c_ptr, _c_int, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
                      _c_ptr],
@@ -263,7 +287,9 @@ _KIND = {"gemm": "matmul", "gemm_mfma": "matmul", "gemm_f32": "matmul", "gemm_pa
          "delta_prep": "attn", "delta_scan": "attn", "delta_out": "attn", "delta_decode": "attn",
          "head_gemm": "matmul", "latent_norm": "attn", "gate_rows": "attn", "gate_heads": "attn",
          "mm_scan": "attn", "mm_chunked": "attn", "mm_out": "attn", "mm_decode": "attn",
-         "lightning_scan": "attn", "lightning_chunked": "attn", "lightning_out": "attn"}
+         "lightning_scan": "attn", "lightning_chunked": "attn", "lightning_out": "attn",
+         "ssd_prep": "attn", "ssd_scan": "attn", "ssd_chunked": "attn", "ssd_decode": "attn", "ssd_out": "attn",
+         "row_norm_kv_write": "attn", "diff_prep_kv_write": "attn", "diff_combine": "attn"}
 
 
 def profile_begin() -> None:
@@ -387,12 +413,14 @@ class GatheredSum:
 
 @dataclasses.dataclass
 class NormedDelta:
-    """A part's output that joins the residual stream only after an RMS norm of its own:
-    ``x += rmsnorm(inner, eps) * weight``, ``inner`` being float32 partial sums [S, T, H] or a GatheredSum.  The next
-    norm does both in one pass; ``materialize`` gives the normed tensor [1, T, H] to whoever needs it earlier."""
+    """A part's output that joins the residual stream only after a norm of its own:
+    ``x += rmsnorm(inner, eps) * weight``, or with ``bias`` ``x += layernorm(inner, eps) * weight + bias``, ``inner`` being
+    float32 partial sums [S, T, H] or a GatheredSum.  The next norm does both in one pass; ``materialize`` gives the normed
+    tensor [1, T, H] to whoever needs it earlier."""
     inner: object
     weight: torch.Tensor
     eps: float
+    bias: torch.Tensor | None = None
 
     def materialize(self, act) -> torch.Tensor:
         ref = self.inner.y if isinstance(self.inner, GatheredSum) else self.inner
@@ -488,9 +516,60 @@ def _add_terms_rmsnorm(x, terms: Terms, weight, eps: float, act, rows, want_act:
     return out, out32
 
 
+def _add_norm(x, delta, weight, bias, eps: float, act, rows, want_act: bool, want_f32: bool, stream: bool):
+    """``add_rmsnorm`` where what is added, or what is returned, passes a layer norm."""
+    k = "add_norm"
+    T, H = x.shape
+    if isinstance(delta, Terms):
+        delta = delta.materialize(act)
+    post = delta if isinstance(delta, NormedDelta) else None
+    inner = post.inner if post is not None else delta
+    y = pair_slot = weights = gate = None
+    topk = 0
+    if isinstance(inner, GatheredSum):
+        y, pair_slot, weights, gate, inner = inner.y, inner.pair_slot, inner.weights, inner.gate, inner.dense
+        _check(y, k, "y", torch.float32)
+        _need(y.dim() == 2 and y.shape[1] == H, k, lambda: f"y must be [rows, {H}]")
+        _check(pair_slot, k, "pair_slot", torch.int32)
+        topk = pair_slot.shape[1]
+        _need(pair_slot.shape[0] == T and 1 <= topk <= 64, k, lambda: f"pair_slot must be [{T}, 1..64]")
+        _check(weights, k, "weights", torch.float32, (T, topk))
+        if gate is not None:
+            _check(gate, k, "gate", torch.float32, (T,))
+    S = 0
+    if inner is not None:
+        _check(inner, k, "delta", torch.float32)
+        _need(inner.dim() == 3 and tuple(inner.shape[1:]) == (T, H), k, lambda: f"delta must be [S, {T}, {H}], is {tuple(inner.shape)}")
+        S = inner.shape[0]
+    wtype = None
+    for name, t in (("the added part's norm weight", post.weight if post is not None else None),
+                    ("the added part's norm bias", post.bias if post is not None else None), ("weight", weight), ("bias", bias)):
+        if t is not None:
+            _check(t, k, name, tuple(_WTYPE), (H,))
+            _need(wtype in (None, t.dtype), k, "the norms' weights and biases must have one type")
+            wtype = t.dtype
+    R = T
+    if rows is not None:
+        _check(rows, k, "rows", torch.int32)
+        _need(rows.dim() == 1 and weight is not None, k, "rows must be [R], and picks rows of what is normed")
+        R = rows.numel()
+    if weight is None:
+        _need(bias is None, k, "a bias goes with a weight")
+        want_act, want_f32 = stream and dtype_name(act) != "float32", False
+    out = torch.empty((R, H), dtype=ACT_DTYPES[dtype_name(act)], device=x.device) if want_act else None
+    out32 = torch.empty((R, H), dtype=torch.float32, device=x.device) if want_f32 else None
+    _run("add_rmsnorm", library(act).tq_add_norm(
+        _ptr(x), _ptr(inner), S, T * H, _ptr(y), _ptr(pair_slot), _ptr(weights), topk, _ptr(gate),
+        0 if post is None else 1 if post.bias is None else 2, _ptr(post.weight) if post is not None else None,
+        _ptr(post.bias) if post is not None else None, float(post.eps) if post is not None else 0.0,
+        0 if weight is None else 1 if bias is None else 2, _ptr(weight), _ptr(bias), float(eps),
+        _WTYPE[wtype] if wtype is not None else 0, _ptr(rows), R, _ptr(out), _ptr(out32), H, _stream()))
+    return (x if stream and out is None else out), out32
+
+
 def add_rmsnorm(x: torch.Tensor, delta, weight: torch.Tensor | None, eps: float, act,
                 rows: torch.Tensor | None = None, want_act: bool = True, want_f32: bool = False, stream: bool = False,
-                shift: tuple | None = None):
+                shift: tuple | None = None, bias: torch.Tensor | None = None):
     """x += delta (in place, unless ``rows`` picks rows), where delta is None, float32 partial sums [S, T, H] added
     one after the other, a GatheredSum, Terms, or a NormedDelta around partial sums or a GatheredSum (then what is added is its RMS norm); returns
     rmsnorm(x) * weight as (activation-typed or None, float32 or None), one row per entry of ``rows`` (all rows if
@@ -499,12 +578,16 @@ def add_rmsnorm(x: torch.Tensor, delta, weight: torch.Tensor | None, eps: float,
     a part that reads the stream un-normed (on the float32 library that is ``x``, which the next sum changes).
     ``shift`` (with ``stream`` behind a NormedDelta, in a step of one token per sequence): (weight float32 [H], state float32
     [slots, H], slots int32 [T]); what is returned is the summed row blended with the row that the sequence's slot keeps,
-    ``a + (state[slot] - a) * weight``, and the slot then keeps the summed row: ``token_shift`` without a launch of its own."""
+    ``a + (state[slot] - a) * weight``, and the slot then keeps the summed row: ``token_shift`` without a launch of its own.
+    ``bias`` (with ``weight``): what is returned is the layer norm of x (the mean taken off), times ``weight``, plus ``bias``."""
     k = "add_rmsnorm"
     _check(x, k, "x", torch.float32)
     _need(x.dim() == 2, k, "x must be [T, H]")
     T, H = x.shape
     post = None
+    if bias is not None or (isinstance(delta, NormedDelta) and delta.bias is not None):
+        _need(shift is None, k, "a shift does not ride behind a layer norm")
+        return _add_norm(x, delta, weight, bias, eps, act, rows, want_act, want_f32, stream)
     if isinstance(delta, Terms):
         _need(not stream and shift is None, k, "the sum of several parts is normed, or only summed")
         return _add_terms_rmsnorm(x, delta, weight, eps, act, rows, want_act, want_f32)
@@ -1221,19 +1304,25 @@ def router_topk(x32: torch.Tensor, router: torch.Tensor, shared_scale: torch.Ten
     ``groups`` (count, keep): only experts of the ``keep`` groups with the largest best score can be chosen.
     ``bias`` float32 [E]: added to the experts' logits before the choice.
     ``sigmoid``: no softmax; an expert's score is the sigmoid of its logit, and the weights are the chosen scores over (their
-    sum + 1e-20), times ``weight_scale`` (``renormalize`` true says so too).  ``pair_groups`` (with it): a group's score is the
+    sum + 1e-20), times ``weight_scale`` (``renormalize`` true says so too).  ``weight_scale`` without it: the softmax over the
+    chosen logits (``renormalize`` true) times that.  ``pair_groups`` (with ``sigmoid``): a group's score is the
     sum of its two largest scores instead of its largest."""
     k = "router_topk"
     T, H, E, ids, weights, gate, logits = _router_outputs(k, x32, router, shared_scale, top_k)
     count, keep = _expert_groups(k, E, top_k, groups, pair_groups)
     if bias is not None:
         _check(bias, k, "bias", torch.float32, (E,))
-    _need(sigmoid or (weight_scale == 1.0 and not pair_groups), k, "a weight scale and groups by their two best go with sigmoid scores")
-    _need(not sigmoid or renormalize, k, "sigmoid scores are renormalised over the chosen")
+    _need(sigmoid or not pair_groups, k, "groups by their two best go with sigmoid scores")
+    _need(not (sigmoid or weight_scale != 1.0) or renormalize, k, "sigmoid scores, and weights with a scale, are renormalised over the chosen")
     if sigmoid:
         _run(k, library(act).tq_router_topk_sigmoid(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype],
                                                     E, top_k, count, keep, int(pair_groups), float(weight_scale), _ptr(ids),
                                                     _ptr(weights), _ptr(gate), _ptr(logits), T, H, _stream()))
+        return ids, weights, gate
+    if weight_scale != 1.0:
+        _run(k, library(act).tq_router_topk_weighted(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype],
+                                                     E, top_k, count, keep, float(weight_scale), _ptr(ids), _ptr(weights),
+                                                     _ptr(gate), _ptr(logits), T, H, _stream()))
         return ids, weights, gate
     _run(k, library(act).tq_router_topk_biased(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E,
                                                top_k, int(bool(renormalize)), count, keep, _ptr(ids), _ptr(weights), _ptr(gate),
@@ -1302,14 +1391,20 @@ def route(x32: torch.Tensor, router: torch.Tensor, shared_scale: torch.Tensor | 
     count, keep = _expert_groups(k, E, top_k, groups, pair_groups)
     if bias is not None:
         _check(bias, k, "bias", torch.float32, (E,))
-    _need(sigmoid or (weight_scale == 1.0 and not pair_groups), k, "a weight scale and groups by their two best go with sigmoid scores")
-    _need(not sigmoid or renormalize, k, "sigmoid scores are renormalised over the chosen")
+    _need(sigmoid or not pair_groups, k, "groups by their two best go with sigmoid scores")
+    _need(not (sigmoid or weight_scale != 1.0) or renormalize, k, "sigmoid scores, and weights with a scale, are renormalised over the chosen")
     cap, sorted_token, pair_slot, tile_expert, n_tiles = _align_outputs(T, top_k, E, unit, x32.device)
     if sigmoid:
         _run(k, library(act).tq_route_sigmoid(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E,
                                               top_k, count, keep, int(pair_groups), float(weight_scale), _ptr(ids), _ptr(weights),
                                               _ptr(gate), _ptr(logits), unit, cap, _ptr(sorted_token), _ptr(pair_slot),
                                               _ptr(tile_expert), _ptr(n_tiles), T, H, _stream()))
+        return ids, weights, gate, sorted_token, pair_slot, tile_expert, n_tiles
+    if weight_scale != 1.0:
+        _run(k, library(act).tq_route_weighted(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E,
+                                               top_k, count, keep, float(weight_scale), _ptr(ids), _ptr(weights), _ptr(gate),
+                                               _ptr(logits), unit, cap, _ptr(sorted_token), _ptr(pair_slot), _ptr(tile_expert),
+                                               _ptr(n_tiles), T, H, _stream()))
         return ids, weights, gate, sorted_token, pair_slot, tile_expert, n_tiles
     _run(k, library(act).tq_route_biased(_ptr(x32), _ptr(router), _ptr(shared_scale), _ptr(bias), _WTYPE[router.dtype], E, top_k,
                                          int(bool(renormalize)), count, keep, _ptr(ids), _ptr(weights), _ptr(gate),
@@ -2038,6 +2133,300 @@ def mm_decode(proj: torch.Tensor, bias: torch.Tensor, runs: dict, state: torch.T
     _run(k, library(act).tq_mm_decode(_ptr(proj), proj.stride(0), _ptr(bias), dims.cap, _ptr(runs["slots"]), _ptr(state),
                                       state.stride(0), B, dims.heads, dims.dim, dims.vdim, _ptr(weight), _WTYPE[weight.dtype],
                                       float(eps), _ptr(out), out.stride(0), *extra, _stream()))
+    return out
+
+
+# ------------------------------------------------------------------ a token's own vector as a factor
+def token_gate(p: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, activation: str, act) -> torch.Tensor:
+    """f(sum_s p[s, t]) * table[tokens[t]] in the activation type: ``p`` float32 [S, T, N] partial sums, ``table`` [V, N], whose
+    rows may be runs of columns of a wider table."""
+    k = "token_gate"
+    _check(p, k, "p", torch.float32)
+    _need(p.dim() == 3, k, "p must be [S, T, N]")
+    S, T, N = p.shape
+    _check(tokens, k, "tokens", torch.int32, (T,))
+    _need(isinstance(table, torch.Tensor) and table.is_cuda and table.dtype in _WTYPE and table.dim() == 2 and table.shape[1] == N
+          and table.stride(1) == 1, k, lambda: f"table must be [V, {N}] on the GPU with unit stride along its rows")
+    out = torch.empty((T, N), dtype=ACT_DTYPES[dtype_name(act)], device=p.device)
+    _run(k, library(act).tq_token_gate(_ptr(p), S, _ptr(tokens), _ptr(table), _WTYPE[table.dtype], table.stride(0),
+                                       _gate_code(k, activation), _ptr(out), T, N, _stream()))
+    return out
+
+
+# ------------------------------------------------------------------ between a product and its attention
+def _kv_places(k: str, k_pages, v_pages, layer_offset: int, page_size: int, page_stride: int, num_kv_heads: int, head_dim: int,
+               block_table, runs, adt):
+    """What a launch that writes keys and values is told: pool addresses, and the runs of a step that brings more than a token
+    per sequence (cu_seqlens, slots, start, number of runs, longest run)."""
+    _check(k_pages, k, "k_pages", adt)
+    _check(v_pages, k, "v_pages", adt)
+    _need(layer_offset + num_kv_heads * page_size * head_dim <= page_stride, k, "layer does not fit in a page")
+    esz = k_pages.element_size()
+    places = (k_pages.data_ptr() + layer_offset * esz, v_pages.data_ptr() + layer_offset * esz)
+    if runs is None or runs["decode"]:
+        return places, (None, None, None, 0, 0)
+    B = runs["slots"].numel()
+    _check(runs["cu_seqlens"], k, "cu_seqlens", torch.int32, (B + 1,))
+    _check(runs["slots"], k, "slots", torch.int32, (B,))
+    _check(runs["start"], k, "start", torch.int32, (B,))
+    _need(int(runs["max_end"]) <= block_table.shape[1] * page_size, k, "positions reach beyond the page table")
+    return places, (_ptr(runs["cu_seqlens"]), _ptr(runs["slots"]), _ptr(runs["start"]), B, int(runs["max_new"]))
+
+
+def _qkv_rows(k: str, qkv, T: int, width: int, head_dim: int) -> None:
+    _need(isinstance(qkv, torch.Tensor) and qkv.is_cuda and qkv.dtype == torch.float32 and qkv.dim() == 2
+          and tuple(qkv.shape) == (T, width) and qkv.stride(1) == 1 and qkv.stride(0) >= width, k,
+          lambda: f"qkv must be float32 [{T}, {width}] on the GPU with unit stride along its rows")
+    _need(head_dim % 4 != 0 or (qkv.stride(0) % 4 == 0 and qkv.data_ptr() % 16 == 0), k,
+          "rows of qkv must start at multiples of 16 bytes")
+
+
+def row_norm_kv_write(qkv: torch.Tensor, positions: torch.Tensor, seq_of_token: torch.Tensor, block_table: torch.Tensor,
+                      inv_freq: torch.Tensor, pairing: int, rotary_dim: int, k_pages: torch.Tensor | None,
+                      v_pages: torch.Tensor | None, layer_offset: int, page_size: int, page_stride: int, num_heads: int,
+                      num_kv_heads: int, head_dim: int, act, q_weight: torch.Tensor, k_weight: torch.Tensor | None, eps: float,
+                      q_dim: int, k_dim: int, values_are_keys: bool = False, runs: dict | None = None,
+                      amplitude: float = 1.0) -> torch.Tensor:
+    """Between the product and the attention where queries and keys are normed over all their heads together: q over all of
+    its numbers (``q_dim`` of them count; heads laid out wider hold zeros) with ``q_weight`` [nh * hd], k alike, then the
+    rotation; keys and values go to the pages, the queries [T, nh * hd] are returned.  ``qkv`` float32 [T, q | k | v]; with
+    ``values_are_keys`` [T, q | k], and the values are the keys as they stand there.  ``k_pages`` None: [T, q], nothing is written."""
+    k = "row_norm_kv_write"
+    T = positions.numel()
+    write = k_pages is not None
+    _qkv_rows(k, qkv, T, (num_heads + (0 if not write else num_kv_heads * (1 if values_are_keys else 2))) * head_dim, head_dim)
+    _check(positions, k, "positions", torch.int32, (T,))
+    _check(seq_of_token, k, "seq_of_token", torch.int32, (T,))
+    _check(block_table, k, "block_table", torch.int32)
+    _need(block_table.dim() == 2, k, "block_table must be [B, pages]")
+    _check(inv_freq, k, "inv_freq", torch.float32)
+    _need(inv_freq.numel() * 2 == rotary_dim or rotary_dim == 0, k, lambda: f"inv_freq must hold rotary_dim/2 = {rotary_dim // 2} entries")
+    _check(q_weight, k, "q_weight", tuple(_WTYPE), (num_heads * head_dim,))
+    if write:
+        _check(k_weight, k, "k_weight", q_weight.dtype, (num_kv_heads * head_dim,))
+    adt = ACT_DTYPES[dtype_name(act)]
+    q = torch.empty((T, num_heads * head_dim), dtype=adt, device=qkv.device)
+    places, tiles = (None, None), (None, None, None, 0, 0)
+    if write:
+        places, tiles = _kv_places(k, k_pages, v_pages, layer_offset, page_size, page_stride, num_kv_heads, head_dim, block_table,
+                                   runs, adt)
+    _run(k, library(act).tq_row_norm_kv_write(
+        _ptr(qkv), qkv.stride(0), _ptr(positions), _ptr(seq_of_token), _ptr(block_table), block_table.shape[1], _ptr(inv_freq),
+        pairing, rotary_dim, float(amplitude), _ptr(q_weight), _ptr(k_weight) if write else None, _WTYPE[q_weight.dtype],
+        float(eps), int(q_dim), int(k_dim), num_heads if values_are_keys else num_heads + num_kv_heads, _ptr(q), *places, page_size,
+        page_stride, T, num_heads, num_kv_heads if write else 0, head_dim, int(write), *tiles, _stream()))
+    return q
+
+
+def diff_prep_kv_write(qkv: torch.Tensor, positions: torch.Tensor, seq_of_token: torch.Tensor, block_table: torch.Tensor,
+                       k_pages: torch.Tensor | None, v_pages: torch.Tensor | None, layer_offset: int, page_size: int,
+                       page_stride: int, num_heads: int, num_kv_heads: int, head_dim: int, act, q_weight: torch.Tensor,
+                       k_weight: torch.Tensor | None, eps: float, norm_dim: int, temperature: tuple[float, float] | None = None,
+                       expand: bool = True, runs: dict | None = None) -> torch.Tensor:
+    """Between the product and a differential attention: ``qkv`` float32 [T, q | k | v], heads of ``head_dim`` numbers, a query
+    or key head being its two maps of head_dim / 2 one behind the other (``norm_dim`` of each count, zeros behind them).  Every
+    map is RMS-normed with ``q_weight`` / ``k_weight`` [head_dim / 2], queries are multiplied by
+    1 + coef ln(floor((position + 1) / every) + 1), ``temperature`` being (coef, every); keys and values go to the pages as rows
+    of head_dim.  Returns the queries: [T, nh * hd], or with ``expand`` [T, 2 nh * hd], each map a head of its own with zeros in
+    the other's place.  ``k_pages`` None: ``qkv`` is [T, q] and nothing is written."""
+    k = "diff_prep_kv_write"
+    T = positions.numel()
+    write = k_pages is not None
+    _need(head_dim % 2 == 0 and 1 <= norm_dim <= head_dim // 2, k, "a head is two maps of half its width")
+    _qkv_rows(k, qkv, T, (num_heads + (2 * num_kv_heads if write else 0)) * head_dim, head_dim)
+    _check(positions, k, "positions", torch.int32, (T,))
+    _check(seq_of_token, k, "seq_of_token", torch.int32, (T,))
+    _check(block_table, k, "block_table", torch.int32)
+    _need(block_table.dim() == 2, k, "block_table must be [B, pages]")
+    _check(q_weight, k, "q_weight", tuple(_WTYPE), (head_dim // 2,))
+    if write:
+        _check(k_weight, k, "k_weight", q_weight.dtype, (head_dim // 2,))
+    coef, every = temperature if temperature is not None else (0.0, 1.0)
+    _need(every > 0, k, "the temperature's step must be positive")
+    adt = ACT_DTYPES[dtype_name(act)]
+    q = torch.empty((T, (2 if expand else 1) * num_heads * head_dim), dtype=adt, device=qkv.device)
+    places, tiles = (None, None), (None, None, None, 0, 0)
+    if write:
+        places, tiles = _kv_places(k, k_pages, v_pages, layer_offset, page_size, page_stride, num_kv_heads, head_dim, block_table,
+                                   runs, adt)
+    _run(k, library(act).tq_diff_prep_kv_write(
+        _ptr(qkv), qkv.stride(0), _ptr(positions), _ptr(seq_of_token), _ptr(block_table), block_table.shape[1], _ptr(q_weight),
+        _ptr(k_weight) if write else None, _WTYPE[q_weight.dtype], float(eps), int(norm_dim), float(coef), float(every), _ptr(q),
+        *places, page_size, page_stride, T, num_heads, num_kv_heads if write else 0, head_dim, int(write), int(expand), *tiles,
+        _stream()))
+    return q
+
+
+def diff_combine(o: torch.Tensor, lam: float, eps: float, value_dim: int, post: float, gate: torch.Tensor | None, num_heads: int,
+                 head_dim: int, act) -> torch.Tensor:
+    """The two maps' outputs of every head made one: r = o[t, 2 h] - lam o[t, 2 h + 1], divided by its root mean square over
+    its first ``value_dim`` numbers, times ``post``, times sigmoid(gate).  ``o`` [T, 2 nh * hd] in the activation type, ``gate``
+    float32 [T, nh * hd] (columns of a wider tensor allowed) or None; returns [T, nh * hd]."""
+    k = "diff_combine"
+    T = o.shape[0]
+    _check(o, k, "o", ACT_DTYPES[dtype_name(act)], (T, 2 * num_heads * head_dim))
+    N = num_heads * head_dim
+    _need(gate is None or (gate.is_cuda and gate.dtype == torch.float32 and tuple(gate.shape) == (T, N) and gate.stride(1) == 1), k,
+          lambda: f"gate must be float32 [{T}, {N}] on the GPU with unit stride along its rows")
+    _need(1 <= value_dim <= head_dim, k, "the values' width lies within the head")
+    out = torch.empty((T, N), dtype=o.dtype, device=o.device)
+    _run(k, library(act).tq_diff_combine(_ptr(o), float(lam), float(eps), int(value_dim), float(post), _ptr(gate),
+                                         gate.stride(0) if gate is not None else 0, _ptr(out), T, num_heads, head_dim, _stream()))
+    return out
+
+
+# ------------------------------------------------------------------ selective state spaces in their dual form
+@dataclasses.dataclass(frozen=True)
+class SsdDims:
+    """Heads, value width, state width, groups and convolution taps of a Mamba-2 mixer."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    taps: int
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        """Channels of the convolution: x, B and C."""
+        return self.inner + 2 * self.groups * self.state
+
+    @property
+    def projections(self) -> int:
+        """Numbers of a token's row of projections: z | x | B | C | dt."""
+        return self.inner + self.channels + self.heads
+
+    @property
+    def state_floats(self) -> int:
+        """Floats of a sequence's row of state: S [heads][state][vdim] and every channel's last taps - 1 inputs, filled up to a
+        multiple of 4."""
+        return -(-(self.heads * self.state * self.vdim + self.channels * (self.taps - 1)) // 4) * 4
+
+    def sizes(self):
+        return self.heads, self.vdim, self.state, self.groups, self.taps
+
+
+def _ssd_proj(k: str, proj: torch.Tensor, d: SsdDims) -> None:
+    _need(isinstance(proj, torch.Tensor) and proj.is_cuda and proj.dtype == torch.float32 and proj.dim() == 2
+          and proj.stride(1) == 1 and proj.shape[1] >= d.projections, k,
+          lambda: f"proj must be float32 [T, >= {d.projections}] on the GPU with unit stride along its rows")
+
+
+def _ssd_state(k: str, state: torch.Tensor, d: SsdDims) -> int:
+    _check(state, k, "state", torch.float32)
+    _need(state.dim() == 2 and state.shape[1] == d.state_floats, k, lambda: f"state must be [slots, {d.state_floats}]")
+    return state.stride(0)
+
+
+def _ssd_runs(k: str, runs: dict) -> int:
+    B = runs["slots"].numel()
+    _check(runs["cu_seqlens"], k, "cu_seqlens", torch.int32, (B + 1,))
+    _check(runs["slots"], k, "slots", torch.int32, (B,))
+    return B
+
+
+def ssd_prep(proj: torch.Tensor, slot_of_token: torch.Tensor, state: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor,
+             dt_bias: torch.Tensor, dims: SsdDims, act):
+    """From the float32 projections [T, z | x | B | C | dt]: x, B and C behind the convolution and silu [T, channels], and
+    softplus(dt + dt_bias) [T, heads].  Inputs before a token's run come from ``state``; nothing is written there."""
+    k = "ssd_prep"
+    T = slot_of_token.numel()
+    _ssd_proj(k, proj, dims)
+    _need(proj.shape[0] == T, k, "a row of projections per token")
+    _check(slot_of_token, k, "slot_of_token", torch.int32, (T,))
+    stride = _ssd_state(k, state, dims)
+    _check(conv_w, k, "conv_w", torch.float32, (dims.channels, dims.taps))
+    _check(conv_b, k, "conv_b", torch.float32, (dims.channels,))
+    _check(dt_bias, k, "dt_bias", torch.float32, (dims.heads,))
+    xbc = torch.empty((T, dims.channels), dtype=torch.float32, device=proj.device)
+    dt = torch.empty((T, dims.heads), dtype=torch.float32, device=proj.device)
+    _run(k, library(act).tq_ssd_prep(_ptr(proj), proj.stride(0), _ptr(slot_of_token), _ptr(state), stride, _ptr(conv_w), _ptr(conv_b),
+                                     _ptr(dt_bias), *dims.sizes(), _ptr(xbc), _ptr(dt), T, _stream()))
+    return xbc, dt
+
+
+def _ssd_rows(k: str, xbc, dt, a_log, skip, d: SsdDims) -> int:
+    T = xbc.shape[0]
+    _check(xbc, k, "xbc", torch.float32, (T, d.channels))
+    _check(dt, k, "dt", torch.float32, (T, d.heads))
+    _check(a_log, k, "a_log", torch.float32, (d.heads,))
+    _check(skip, k, "skip", torch.float32, (d.heads,))
+    return T
+
+
+def ssd_scan(xbc: torch.Tensor, dt: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor, runs: dict, state: torch.Tensor,
+             dims: SsdDims, act) -> torch.Tensor:
+    """S <- exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + skip x over the step's runs of tokens, in order, from and into the
+    sequences' rows of ``state``.  Returns y float32 [T, heads * vdim]."""
+    k = "ssd_scan"
+    T = _ssd_rows(k, xbc, dt, a_log, skip, dims)
+    stride = _ssd_state(k, state, dims)
+    _need(dims.state <= 1024, k, lambda: f"a state of {dims.state} channels is beyond the 1,024 this kernel takes")
+    B = _ssd_runs(k, runs)
+    y = torch.empty((T, dims.inner), dtype=torch.float32, device=xbc.device)
+    _run(k, library(act).tq_ssd_scan(_ptr(xbc), _ptr(dt), _ptr(a_log), _ptr(skip), _ptr(runs["cu_seqlens"]), _ptr(runs["slots"]),
+                                     _ptr(state), stride, *dims.sizes(), B, _ptr(y), _stream()))
+    return y
+
+
+def ssd_chunked(xbc: torch.Tensor, dt: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor, runs: dict, state: torch.Tensor,
+                dims: SsdDims, act) -> torch.Tensor:
+    """``ssd_scan`` for steps with long runs: the same sums over chunks of 64 tokens on the matrix cores, in float32 on both
+    libraries (three launches), states of up to 256 channels.  ``runs`` also names ``max_new``, the longest run."""
+    k = "ssd_chunked"
+    T = _ssd_rows(k, xbc, dt, a_log, skip, dims)
+    stride = _ssd_state(k, state, dims)
+    _need(dims.state <= 256, k, lambda: f"a state of {dims.state} channels is beyond the 256 this kernel takes")
+    B, max_new = _ssd_runs(k, runs), int(runs["max_new"])
+    _need(1 <= max_new <= T, k, lambda: f"the longest run has {max_new} of {T} tokens")
+    chunks = T // LIGHTNING_CHUNK + B
+    scratch = torch.empty((chunks, dims.inner * dims.state), dtype=torch.float32, device=xbc.device)
+    tot = torch.empty((chunks, dims.heads), dtype=torch.float32, device=xbc.device)
+    y = torch.empty((T, dims.inner), dtype=torch.float32, device=xbc.device)
+    _run(k, library(act).tq_ssd_chunked(_ptr(xbc), _ptr(dt), _ptr(a_log), _ptr(skip), _ptr(runs["cu_seqlens"]), _ptr(runs["slots"]),
+                                        _ptr(state), stride, *dims.sizes(), B, max_new, _ptr(scratch), _ptr(tot), chunks, _ptr(y),
+                                        _stream()))
+    return y
+
+
+def ssd_decode(proj: torch.Tensor, runs: dict, state: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor,
+               dt_bias: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor, dims: SsdDims, act) -> torch.Tensor:
+    """``ssd_prep`` and ``ssd_scan`` of a step of one token per sequence, in one launch (``ssd_out`` moves the convolution's
+    state on).  Returns y float32 [B, heads * vdim]."""
+    k = "ssd_decode"
+    _ssd_proj(k, proj, dims)
+    stride = _ssd_state(k, state, dims)
+    B = _ssd_runs(k, runs)
+    _need(proj.shape[0] == B and runs["decode"], k, "decoding brings one token per sequence")
+    _check(conv_w, k, "conv_w", torch.float32, (dims.channels, dims.taps))
+    for name, t, n in (("conv_b", conv_b, dims.channels), ("dt_bias", dt_bias, dims.heads), ("a_log", a_log, dims.heads),
+                       ("skip", skip, dims.heads)):
+        _check(t, k, name, torch.float32, (n,))
+    y = torch.empty((B, dims.inner), dtype=torch.float32, device=proj.device)
+    _run(k, library(act).tq_ssd_decode(_ptr(proj), proj.stride(0), _ptr(runs["slots"]), _ptr(state), stride, _ptr(conv_w), _ptr(conv_b),
+                                       _ptr(dt_bias), _ptr(a_log), _ptr(skip), *dims.sizes(), B, _ptr(y), _stream()))
+    return y
+
+
+def ssd_out(y: torch.Tensor, proj: torch.Tensor, weight: torch.Tensor, eps: float, parts: int, runs: dict, state: torch.Tensor,
+            dims: SsdDims, act) -> torch.Tensor:
+    """y silu(z) divided by its root mean square in ``parts`` equal parts, times ``weight`` [heads * vdim], in the activation
+    type (z: the first columns of ``proj``); and the convolution's part of every sequence's state brought to its run's end."""
+    k = "ssd_out"
+    T = y.shape[0]
+    _check(y, k, "y", torch.float32, (T, dims.inner))
+    _ssd_proj(k, proj, dims)
+    _need(proj.shape[0] == T and parts >= 1 and dims.inner % parts == 0, k, "a row of projections per token, and equal parts")
+    _check(weight, k, "weight", tuple(_WTYPE), (dims.inner,))
+    stride = _ssd_state(k, state, dims)
+    B = _ssd_runs(k, runs)
+    out = torch.empty((T, dims.inner), dtype=ACT_DTYPES[dtype_name(act)], device=y.device)
+    _run(k, library(act).tq_ssd_out(_ptr(y), _ptr(proj), proj.stride(0), _ptr(weight), _WTYPE[weight.dtype], float(eps), int(parts),
+                                    _ptr(runs["cu_seqlens"]), _ptr(runs["slots"]), _ptr(state), stride, *dims.sizes(), T, B,
+                                    _ptr(out), _stream()))
     return out
 
 

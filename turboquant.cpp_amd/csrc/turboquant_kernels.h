@@ -204,6 +204,49 @@ int tq_router_topk_sigmoid(const float* x, const void* wr, const void* shared_w,
 int tq_route_sigmoid(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E, int topk,
         int groups, int keep, int pair_groups, float wscale, int* ids, float* weights, float* shared_gate, float* logits,
         int unit, int cap, int* sorted_token, int* pair_slot, int* tile_expert, int* n_tiles, int T, int H, hipStream_t st);
+// Weights are the softmax over the chosen experts' logits, times wscale.
+int tq_router_topk_weighted(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E,
+        int topk, int groups, int keep, float wscale, int* ids, float* weights, float* shared_gate, float* logits, int T,
+        int H, hipStream_t st);
+int tq_route_weighted(const float* x, const void* wr, const void* shared_w, const float* bias, int wtype, int E, int topk,
+        int groups, int keep, float wscale, int* ids, float* weights, float* shared_gate, float* logits, int unit, int cap,
+        int* sorted_token, int* pair_slot, int* tile_expert, int* n_tiles, int T, int H, hipStream_t st);
+// add_layernorm.hip: residual sum with norms that may take the mean off; token_gate.hip: a token's own vector as a factor
+int tq_add_norm(float* x, const float* delta, int S, int64_t delta_stride, const float* y, const int* pair_slot,
+        const float* weights, int topk, const float* gate, int kind_d, const void* wd, const void* bd, float eps_d,
+        int kind, const void* w, const void* b, float eps, int wtype, const int* rows, int R, void* out, float* out32,
+        int H, hipStream_t st);
+int tq_token_gate(const float* p, int S, const int* tokens, const void* table, int wtype, int64_t ld_table, int kind,
+        void* out, int T, int N, hipStream_t st);
+// attention_prep.hip: between a product and its attention; two maps a head made one
+int tq_row_norm_kv_write(const float* qkv, int64_t ld, const int* positions, const int* seq_of_token,
+        const int* block_table, int bt_stride, const float* inv_freq, int pairing, int rot, float amp, const void* wq,
+        const void* wk, int wtype, float eps, int q_dim, int k_dim, int first_value, void* q_out, void* k_pool,
+        void* v_pool, int page_size, int64_t page_stride, int T, int nh, int nkv, int hd, int write_kv,
+        const int* cu_seqlens, const int* slots, const int* start, int B, int max_new, hipStream_t st);
+int tq_diff_prep_kv_write(const float* qkv, int64_t ld, const int* positions, const int* seq_of_token,
+        const int* block_table, int bt_stride, const void* wq, const void* wk, int wtype, float eps, int norm_dim,
+        float coef, float every, void* q_out, void* k_pool, void* v_pool, int page_size, int64_t page_stride, int T, int nh,
+        int nkv, int hd, int write_kv, int expand, const int* cu_seqlens, const int* slots, const int* start, int B,
+        int max_new, hipStream_t st);
+int tq_diff_combine(const void* o, float lambda, float eps, int vd, float post, const float* gate, int64_t ld_gate,
+        void* out, int T, int nh, int hd, hipStream_t st);
+// ssd.hip: selective state spaces in their dual form (Mamba-2)
+int tq_ssd_prep(const float* P, int64_t ldp, const int* slot_of_token, const float* state, int64_t state_stride,
+        const float* conv_w, const float* conv_b, const float* dt_bias, int H, int V, int N, int G, int taps, float* xbc,
+        float* dt, int T, hipStream_t st);
+int tq_ssd_scan(const float* xbc, const float* dt, const float* a_log, const float* D, const int* cu_seqlens,
+        const int* slots, float* state, int64_t state_stride, int H, int V, int N, int G, int taps, int B, float* y,
+        hipStream_t st);
+int tq_ssd_chunked(const float* xbc, const float* dt, const float* a_log, const float* D, const int* cu_seqlens,
+        const int* slots, float* state, int64_t state_stride, int H, int V, int N, int G, int taps, int B, int max_new,
+        float* scratch, float* tot, int chunks, float* y, hipStream_t st);
+int tq_ssd_decode(const float* P, int64_t ldp, const int* slots, float* state, int64_t state_stride, const float* conv_w,
+        const float* conv_b, const float* dt_bias, const float* a_log, const float* D, int H, int V, int N, int G, int taps,
+        int B, float* y, hipStream_t st);
+int tq_ssd_out(const float* y, const float* P, int64_t ldp, const void* w, int wtype, float eps, int parts,
+        const int* cu_seqlens, const int* slots, float* state, int64_t state_stride, int H, int V, int N, int G, int taps,
+        int T, int B, void* out, hipStream_t st);
 // The *_sig forms of the attention entry points add what score_mod.h calls pb and keep: sigmoid weights with a bias per
 // head in the softmax's place, and first positions that stay visible whatever the window.
 int tq_attention_generic_sig(const void* q, const void* k_pool, const void* v_pool, const int* positions,

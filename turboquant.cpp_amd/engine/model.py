@@ -79,6 +79,10 @@ class CausalLM:
         if plan.position_table is not None:
             self.bindings.append(Binding(self, "position_table", ParamSpec((plan.max_positions, H), role="table"),
                                          plan.position_table, "position_table"))
+        self.token_table = None        # [V, n]: a second row per token, whose columns the layers' side parts share out
+        if plan.token_table is not None:
+            self.bindings.append(Binding(self, "token_table", ParamSpec((V, plan.token_table_width), role="table"),
+                                         plan.token_table, "token_table"))
         self.step_vectors = None       # [n, H] float32: vectors that schedule entries add to the stream
         if plan.step_vectors is not None:
             self.bindings.append(Binding(self, "step_vectors", ParamSpec((plan.n_step_vectors, H), role="bias"),
@@ -99,6 +103,8 @@ class CausalLM:
         if self.step_vectors is not None:
             self.step_vectors = self.step_vectors.float().contiguous()      # they enter float arithmetic only
         for part in self.parts():
+            if self.token_table is not None and hasattr(part, "token_columns"):
+                part.token_rows = self.token_table[:, part.token_columns[0]:part.token_columns[1]]
             part.prepare(self.device, self.act)
         return self
 

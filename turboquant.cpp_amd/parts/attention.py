@@ -27,6 +27,9 @@ step; "mix": its values become (1 - mix) v + mix v_source, ``mix`` a learned num
 carry the parameter, which a source does not use); ``sigmoid_bias`` (no softmax: the weight of a visible key is
 sigmoid(score + b_h), b a learned number per head, and the weights are not normalised over the keys); ``keep_first`` n
 (with a window: the sequence's first n positions stay visible to every later token and stay in the cache).
+``row_norm_eps`` (queries and keys are RMS-normed before the rotation over all their heads together, with a weight per number
+of the whole projection); ``values_are_keys`` (there is no value matrix: the values are the keys as they were projected, before
+norm and rotation); ``unit_sink`` (the softmax's denominator also holds 1: a sink whose score is 0, the same for every head).
 With ``separate_qkv`` the heads are laid out at a kernel width that is the larger of key and value width rounded up to
 16: the added rows and columns of the matrices are zeros, which change no score and no output, and every head size
 then runs on the matrix-core kernels of both libraries.
@@ -52,7 +55,17 @@ class GroupedQueryAttention(Part):
                  separate_qkv: bool = False, sink: bool = False, rotated_norm_eps: float | None = None,
                  head_gate: bool = False, shares_kv: bool = False, cache_window: int | None | str = "own",
                  value_norm_eps: float | None = None, value_mix: str | None = None, sigmoid_bias: bool = False,
-                 keep_first: int = 0):
+                 keep_first: int = 0, row_norm_eps: float | None = None, values_are_keys: bool = False, unit_sink: bool = False):
+        if (row_norm_eps is not None or values_are_keys or unit_sink) and not separate_qkv:
+            raise ValueError("a norm over all heads, values that are the keys and a sink of one need separate_qkv")
+        if row_norm_eps is not None and (not row_norm_eps > 0 or qk_norm_eps is not None or rotated_norm_eps is not None
+                                         or value_norm_eps is not None or value_mix is not None or head_gate or qkv_bias):
+            raise ValueError("a norm over all heads has a positive eps and comes without other norms, gates and biases")
+        if values_are_keys and (row_norm_eps is None or value_dim not in (None, head_dim)):
+            raise ValueError("values that are the keys are as wide as these, and go with a norm over all heads")
+        if unit_sink and (sink or sigmoid_bias):
+            raise ValueError("a sink of one goes with a softmax without another sink")
+        self.row_norm_eps, self.values_are_keys, self.unit_sink = row_norm_eps, values_are_keys, unit_sink
         if value_mix not in (None, "source", "mix"):
             raise ValueError(f"value_mix is None, 'source' or 'mix', got {value_mix!r}")
         if (value_norm_eps is not None or value_mix is not None or sigmoid_bias or keep_first) and not separate_qkv:
@@ -116,7 +129,13 @@ class GroupedQueryAttention(Part):
             H, G, K, V, W = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim, self.hidden_size
             specs = {"q_weight": ParamSpec((H * K, W)), "out_weight": ParamSpec((W, H * V))}
             if not self.shares_kv:
-                specs.update({"k_weight": ParamSpec((G * K, W)), "v_weight": ParamSpec((G * V, W))})
+                specs["k_weight"] = ParamSpec((G * K, W))
+                if not self.values_are_keys:
+                    specs["v_weight"] = ParamSpec((G * V, W))
+            if self.row_norm_eps is not None:
+                specs["q_norm"] = ParamSpec((H * K,), role="scale")
+                if not self.shares_kv:
+                    specs["k_norm"] = ParamSpec((G * K,), role="scale")
             if self.has_head_gate:
                 specs["gate_weight"] = ParamSpec((H, W))
             if self.has_qkv_bias:
@@ -164,6 +183,8 @@ class GroupedQueryAttention(Part):
             self.score_bias = self.score_bias.float().contiguous()
         if self.value_mix is not None:
             self.mix = self.mix.reshape(1).contiguous()
+        if self.unit_sink and self.sink is None:
+            self.sink = torch.zeros((self.num_heads,), dtype=torch.float32, device=device)
         if not self.separate_qkv or self.qkv_weight is not None:
             return
         D = self.head_dim
@@ -177,9 +198,14 @@ class GroupedQueryAttention(Part):
         H, G, K, V = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
         if self.qk_norm_eps is not None and K != D:     # zeros behind the head's own values: they norm zeros to zeros
             self.q_norm, self.k_norm = (torch.cat([w, w.new_zeros(D - K)]) for w in (self.q_norm, self.k_norm))
+        if self.row_norm_eps is not None:
+            self.q_norm = heads_padded(self.q_norm, H, K).contiguous()
+            self.k_norm = None if self.shares_kv else heads_padded(self.k_norm, G, K).contiguous()
         rows = [heads_padded(self.q_weight, H, K)]
         if not self.shares_kv:
-            rows += [heads_padded(self.k_weight, G, K), heads_padded(self.v_weight, G, V)]
+            rows.append(heads_padded(self.k_weight, G, K))
+            if not self.values_are_keys:
+                rows.append(heads_padded(self.v_weight, G, V))
         if self.has_head_gate:      # the gate's rows ride in the same product, filled up to a multiple of four rows
             fill = -H % 4
             rows += [self.gate_weight, self.gate_weight.new_zeros((fill, self.hidden_size))]
@@ -233,7 +259,7 @@ class GroupedQueryAttention(Part):
             opts["distance_bias"] = (self.r1, self.r2)
         if self.chunk is not None:
             opts["chunk"] = self.chunk
-        if self.has_sink:
+        if self.has_sink or self.unit_sink:
             opts["sink"] = self.sink
         if self.has_sigmoid_bias:
             opts["sigmoid_bias"] = self.score_bias
@@ -246,7 +272,7 @@ class GroupedQueryAttention(Part):
         """The matrix of q, k and v where nothing but the product stands between the input and the rotation, else None."""
         if (not self.separate_qkv or self.qkv_bias is not None or self.qk_norm_eps is not None or self.rotated_norm_eps is not None
                 or self.has_head_gate or self.shares_kv or self.value_norm_eps is not None or self.value_mix is not None
-                or getattr(self.position, "amplitude", 1.0) != 1.0):
+                or self.row_norm_eps is not None or getattr(self.position, "amplitude", 1.0) != 1.0):
             return None
         return self.qkv_weight
 
@@ -286,6 +312,8 @@ class GroupedQueryAttention(Part):
     def forward(self, normed, ctx, entry):
         b, kv = ctx.batch, ctx.kv(entry)
         amplitude = getattr(self.position, "amplitude", 1.0)
+        if self.row_norm_eps is not None:
+            return self._forward_row_norm(normed, ctx, b, kv, amplitude)
         if (self.rotated_norm_eps is not None or self.has_head_gate or self.shares_kv or amplitude != 1.0
                 or self.value_norm_eps is not None or self.value_mix is not None):
             return self._forward_extended(normed, ctx, b, kv, amplitude)
@@ -302,6 +330,22 @@ class GroupedQueryAttention(Part):
         o = ops.attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table,
                           kv.page_size, kv.page_stride, self.num_heads, self.num_kv_heads, self.head_dim,
                           self.window, self.scale, ctx.act, runs=b.runs(), **self._score_options())
+        return ops.gemm(o, self.out_weight, ctx.act, bias=self.out_bias, partial_sums=True)
+
+    def _forward_row_norm(self, normed, ctx, b, kv, amplitude):
+        """The form with a norm over all heads: one product (q | k | v, or q | k where the values are the keys), norms, rotation
+        and cache write in one launch, attention, the output product."""
+        if kv.owns == self.shares_kv:
+            raise ValueError("an attention keeps a cache of its own exactly if it has keys and values of its own")
+        H, G, D = self.num_heads, self.num_kv_heads, self.head_dim
+        qkv = ops.gemm(normed, self.qkv_weight, ctx.act)
+        q = ops.row_norm_kv_write(qkv, b.positions, b.slot_of_token, kv.table, self.position.table(ctx.device),
+                                  self.position.pairing_code, self.position.rotary_dim, kv.k_pages if kv.owns else None,
+                                  kv.v_pages if kv.owns else None, kv.layer_offset, kv.page_size, kv.page_stride, H, G, D, ctx.act,
+                                  self.q_norm, self.k_norm, self.row_norm_eps, H * self.key_dim, G * self.key_dim,
+                                  values_are_keys=self.values_are_keys, runs=b.runs(), amplitude=amplitude)
+        o = ops.attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table, kv.page_size,
+                          kv.page_stride, H, G, D, self.window, self.scale, ctx.act, runs=b.runs(), **self._score_options())
         return ops.gemm(o, self.out_weight, ctx.act, bias=self.out_bias, partial_sums=True)
 
     def _forward_extended(self, normed, ctx, b, kv, amplitude):

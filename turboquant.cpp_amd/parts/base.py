@@ -20,6 +20,9 @@ Interfaces (``ctx`` is the :class:`~..engine.context.StepContext` of the running
 * ffn       ``forward(normed, normed32, ctx) -> delta``; ``wants_f32`` says whether it reads the float32 copy.
 * shift     ``forward(x, ctx, entry) -> h``: what a mixer reads of the float32 stream ``x`` where every token is blended with
             the one before it; ``state_need()`` says what it keeps per sequence between steps.
+* side      ``forward(h, ctx) -> pending``: what a layer adds to the stream last, from the stream ``h`` in the activation type
+            and the tokens' own vectors, which it finds in ``token_rows`` (the model sets it: columns ``token_columns`` of the
+            model's table with a row per token of the vocabulary).
 * position  ``table(device)``, ``pairing``, ``rotary_dim``: the rotation a mixer applies to queries and keys.
 * block     ``forward(x, pending, ctx, entry) -> pending``: the arrangement of norms, mixer and ffn around
             the residual stream.
@@ -109,7 +112,7 @@ class Part:
 
 
 _REGISTRIES: dict[str, dict[str, Callable[..., Part]]] = {
-    "norm": {}, "mixer": {}, "ffn": {}, "position": {}, "block": {}, "shift": {},
+    "norm": {}, "mixer": {}, "ffn": {}, "position": {}, "block": {}, "shift": {}, "side": {},
 }
 
 

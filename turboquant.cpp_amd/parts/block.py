@@ -9,6 +9,7 @@ from __future__ import annotations
 
 import torch
 
+from ..csrc import ops
 from .base import Part, register_part
 
 
@@ -74,7 +75,6 @@ class ParallelBlock(Part):
         return self.mixer.state_need()
 
     def forward(self, x, pending, ctx, entry):
-        from ..csrc import ops
         normed, normed32 = self.norm.forward(x, pending, ctx, want_f32=getattr(self.ffn, "wants_f32", False))
         mixed = self.mixer.forward(normed, ctx, entry)
         fed = None if self.ffn is None else self.ffn.forward(normed, normed32, ctx)
@@ -110,14 +110,13 @@ class SandwichBlock(Part):
         return self.mixer.state_need()
 
     def forward(self, x, pending, ctx, entry):
-        from ..csrc import ops
         normed, _ = self.mixer_norm.forward(x, pending, ctx)
-        pending = ops.NormedDelta(self.mixer.forward(normed, ctx, entry), self.mixer_post_norm.weight, self.mixer_post_norm.eps)
+        pending = self.mixer_post_norm.over(self.mixer.forward(normed, ctx, entry))
         if self.ffn is None:
             return pending
         want32 = getattr(self.ffn, "wants_f32", False)
         normed, normed32 = self.ffn_norm.forward(x, pending, ctx, want_f32=want32)
-        return ops.NormedDelta(self.ffn.forward(normed, normed32, ctx), self.ffn_post_norm.weight, self.ffn_post_norm.eps)
+        return self.ffn_post_norm.over(self.ffn.forward(normed, normed32, ctx))
 
 
 @register_part("block", "outnorm")
@@ -129,21 +128,24 @@ class OutputNormBlock(Part):
     ``mixer_shift`` (optional, a part of the "shift" registry): the mixer reads the stream blended token by token with the
     row before (``parts/shift.py``) instead of the stream itself; the feed-forward still reads the stream.  What the shift
     keeps per sequence is the layer's state, so it goes with mixers that keep none of their own.  A feed-forward that wants
-    its input in float32 as well (a router) is given the stream itself."""
+    its input in float32 as well (a router) is given the stream itself.
+    ``side`` (optional, a part of the "side" registry): what the layer adds to the stream last, from the stream behind the
+    feed-forward and the token's own vector."""
     graph_safe = True
-    slots = {"mixer": "mixer", "mixer_norm": "norm", "ffn": "ffn", "ffn_norm": "norm", "mixer_shift": "shift"}
-    optional = ("ffn", "ffn_norm", "mixer_shift")
+    slots = {"mixer": "mixer", "mixer_norm": "norm", "ffn": "ffn", "ffn_norm": "norm", "mixer_shift": "shift", "side": "side"}
+    optional = ("ffn", "ffn_norm", "mixer_shift", "side")
 
-    def __init__(self, mixer, mixer_norm, ffn=None, ffn_norm=None, mixer_shift=None):
+    def __init__(self, mixer, mixer_norm, ffn=None, ffn_norm=None, mixer_shift=None, side=None):
         if (ffn is None) != (ffn_norm is None):
             raise ValueError("a layer has a feed-forward with its norm, or neither")
         if mixer_shift is not None and mixer.state_need() is not None:
             raise ValueError("a shifted input goes with a mixer that keeps no state of its own per sequence")
         self.mixer, self.mixer_norm, self.ffn, self.ffn_norm, self.mixer_shift = mixer, mixer_norm, ffn, ffn_norm, mixer_shift
+        self.side = side
 
     def children(self):
         parts = {"mixer": self.mixer, "mixer_norm": self.mixer_norm, "ffn": self.ffn, "ffn_norm": self.ffn_norm,
-                 "mixer_shift": self.mixer_shift}
+                 "mixer_shift": self.mixer_shift, "side": self.side}
         return {k: v for k, v in parts.items() if v is not None}
 
     def cache_need(self):
@@ -153,7 +155,6 @@ class OutputNormBlock(Part):
         return self.mixer.state_need() if self.mixer_shift is None else self.mixer_shift.state_need()
 
     def forward(self, x, pending, ctx, entry):
-        from ..csrc import ops
         if pending is not None and not isinstance(pending, ops.NormedDelta):     # a layer of another arrangement before this one
             ops.add_rmsnorm(x, pending, self.mixer_norm.weight, self.mixer_norm.eps, ctx.act, want_act=False)
             pending = None
@@ -167,11 +168,17 @@ class OutputNormBlock(Part):
                 if pending is not None:
                     ops.add_rmsnorm(x, pending, None, 0.0, ctx.act)
                 h = self.mixer_shift.forward(x, ctx, entry)
-        pending = ops.NormedDelta(self.mixer.forward(h, ctx, entry), self.mixer_norm.weight, self.mixer_norm.eps)
+        pending = self.mixer_norm.over(self.mixer.forward(h, ctx, entry))
         if self.ffn is None:
-            return pending
+            return self._with_side(x, pending, ctx)
         h, _ = ops.add_rmsnorm(x, pending, None, 0.0, ctx.act, stream=True)
         # (a feed-forward that reads float32 rows reads the stream; what it hands on may name those rows, and the kernel
         # that sums it into the stream reads a row whole before it writes that row)
-        return ops.NormedDelta(self.ffn.forward(h, x if getattr(self.ffn, "wants_f32", False) else None, ctx),
-                               self.ffn_norm.weight, self.ffn_norm.eps)
+        pending = self.ffn_norm.over(self.ffn.forward(h, x if getattr(self.ffn, "wants_f32", False) else None, ctx))
+        return self._with_side(x, pending, ctx)
+
+    def _with_side(self, x, pending, ctx):
+        if self.side is None:
+            return pending
+        h, _ = ops.add_rmsnorm(x, pending, None, 0.0, ctx.act, stream=True)
+        return self.side.forward(h, ctx)

@@ -3,7 +3,7 @@ experts and a shared expert.
 
 Dense (/root/reference/src/engine/tq_transformer.c:2707-2824): ``down(silu(gate x) * (up x))``, no biases; the
 gate's activation is an argument (``silu``, ``gelu_tanh`` as /root/reference/src/engine/tq_ops.c:1482-1484, ``relu2``)
-that the products' epilogues take.
+that the products' epilogues take.  ``pair_limit`` L: ``down(f(min(gate x, L)) * (clamp(up x, -L, L) + 1))``.
 Sparse (/root/reference/src/engine/tq_moe.c:600-1059): router logits in float32, top-k with the highest index
 winning ties, weights from a softmax; every chosen expert is the dense formula with its own matrices, summed
 with its weight in the order chosen; the shared expert, scaled by ``sigmoid(x . shared_scale)``, is added
@@ -12,7 +12,8 @@ the reference's softmax over the chosen logits.  ``router_bias``: a number per e
 choice.  ``pair_limit`` L: an expert is ``down(f(min(gate x, L)) * (clamp(up x, -L, L) + 1))``.  ``groups`` (count, keep): the experts form ``count`` equal groups of
 neighbours, a group's score is the largest score in it (``pair_groups``: the sum of its two largest), and only experts of
 the ``keep`` best groups can be chosen.  ``sigmoid_scores``: an expert's score is the sigmoid of its logit, the choice is by
-score, and the weights are the chosen scores over (their sum + 1e-20), times ``weight_scale``.  ``shared_limit`` L: the
+score, and the weights are the chosen scores over (their sum + 1e-20), times ``weight_scale`` (which the softmax over the
+chosen logits may have too).  ``shared_limit`` L: the
 shared expert's pair is clamped as ``pair_limit`` clamps the experts' (the two may differ).
 ``gated`` false: an expert is ``down(f(up x))``, two matrices and no gate.  ``score_correction``: the softmax runs over all
 of the router's rows, the choice is by score plus a learned number per row, and the weights are the scores themselves,
@@ -40,10 +41,12 @@ class DenseSwiGLU(Part):
     graph_safe = True
     wants_f32 = False
 
-    def __init__(self, hidden_size: int, inner_size: int, activation: str = "silu"):
+    def __init__(self, hidden_size: int, inner_size: int, activation: str = "silu", pair_limit: float | None = None):
         if activation not in ops.GATES:
             raise ValueError(f"unknown activation {activation!r}; known: {', '.join(sorted(ops.GATES))}")
-        self.hidden_size, self.inner_size, self.activation = hidden_size, inner_size, activation
+        if pair_limit is not None and not pair_limit > 0:
+            raise ValueError(f"pair_limit must be positive, got {pair_limit}")
+        self.hidden_size, self.inner_size, self.activation, self.pair_limit = hidden_size, inner_size, activation, pair_limit
         self.gate = self.up = self.down = None
 
     def param_specs(self):
@@ -57,11 +60,14 @@ class DenseSwiGLU(Part):
 
     def native(self):
         from ..csrc import host_api
+        if self.pair_limit is not None:
+            return None                  # the executor's pairs have no limit
         return host_api.DenseFfnDesc(self.hidden_size, self.inner_size, ops.GATES[self.activation], host_api.weight(self.gate),
                                      host_api.weight(self.up), host_api.weight(self.down))
 
     def forward(self, normed, normed32, ctx):
-        h = ops.gemm(normed, self.gate, ctx.act, w2=self.up, out_act=True, activation=self.activation)
+        h = ops.gemm(normed, self.gate, ctx.act, w2=self.up, out_act=True, activation=self.activation,
+                     **({} if self.pair_limit is None else {"pair_limit": self.pair_limit}))
         return ops.gemm(h, self.down, ctx.act, partial_sums=True)
 
 
@@ -99,8 +105,10 @@ class SparseMoE(Part):
                  weight_scale: float = 1.0, pair_groups: bool = False, shared_limit: float | None = None):
         if sigmoid_scores and (score_correction or not renormalize or not gated):
             raise ValueError("sigmoid scores are renormalised over the chosen experts, which are gated pairs, and come without a correction")
-        if not sigmoid_scores and (weight_scale != 1.0 or pair_groups):
-            raise ValueError("a weight scale and groups by their two best scores go with sigmoid scores")
+        if not sigmoid_scores and pair_groups:
+            raise ValueError("groups by their two best scores go with sigmoid scores")
+        if weight_scale != 1.0 and (not renormalize or score_correction or not gated):
+            raise ValueError("a weight scale goes with weights renormalised over the chosen experts, which are gated pairs")
         if shared_limit is not None and not (shared_size > 0 and shared_limit > 0):
             raise ValueError(f"shared_limit is for a shared expert and positive, got {shared_limit}")
         self.sigmoid_scores, self.weight_scale, self.pair_groups = sigmoid_scores, float(weight_scale), bool(pair_groups)
@@ -163,7 +171,7 @@ class SparseMoE(Part):
         from ..csrc import host_api
         w = host_api.weight
         if (self.groups is not None or self.has_router_bias or self.pair_limit is not None or not self.gated or self.score_correction
-                or self.sigmoid_scores or self.shared_limit is not None):
+                or self.sigmoid_scores or self.shared_limit is not None or self.weight_scale != 1.0):
             return None                  # the executor chooses among all experts, by logits without a bias, for plain pairs
         return host_api.MoeFfnDesc(self.hidden_size, self.num_experts, self.top_k, self.expert_size, self.shared_size,
                                    int(self.renormalize), ops.GATES[self.activation], w(self.router),
@@ -180,8 +188,8 @@ class SparseMoE(Part):
                                   self.top_k, self.renormalize, unit, ctx.act,
                                   **({} if self.groups is None else {"groups": self.groups}),
                                   **({} if self.router_bias is None else {"bias": self.router_bias}),
-                                  **({} if not self.sigmoid_scores else {"sigmoid": True, "weight_scale": self.weight_scale,
-                                                                         "pair_groups": self.pair_groups}))
+                                  **({} if self.weight_scale == 1.0 else {"weight_scale": self.weight_scale}),
+                                  **({} if not self.sigmoid_scores else {"sigmoid": True, "pair_groups": self.pair_groups}))
         limit = {} if self.pair_limit is None else {"pair_limit": self.pair_limit}
         if self.shared_size > 0 and T <= 16 and unit == 16:
             # a handful of tokens: the shared expert's two products ride in the launches of the routed experts'

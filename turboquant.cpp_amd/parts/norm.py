@@ -1,4 +1,4 @@
-"""RMS norm fused with the sum into the residual stream.
+"""Norms fused with the sum into the residual stream: the RMS norm, and the layer norm at the end of this file.
 
 ``out = (v * (1 / sqrt(mean(v^2) + eps))) * weight`` with ``v = x + pending``, everything in float32
 (/root/reference/src/engine/tq_ops.c:1373-1410; a plain weight, no ``+1``).
@@ -33,6 +33,34 @@ class RMSNorm(Part):
         from ..csrc import host_api
         return host_api.NormDesc(host_api.weight(self.weight), self.eps)
 
+    def over(self, inner) -> ops.NormedDelta:
+        """What a part left for the stream, to pass this norm as it is added."""
+        return ops.NormedDelta(inner, self.weight, self.eps)
+
     def forward(self, x, delta, ctx, rows=None, want_act=True, want_f32=False):
         return ops.add_rmsnorm(x, delta, self.weight, self.eps, ctx.act, rows=rows, want_act=want_act,
                                want_f32=want_f32)
+
+
+@register_part("norm", "layernorm")
+class LayerNorm(Part):
+    """``out = (v - mean(v)) * (1 / sqrt(mean((v - mean(v))^2) + eps)) * weight + bias`` with ``v = x + pending``, in float32;
+    the weights and the bias enter float32 arithmetic only and are kept in it."""
+    graph_safe = True
+
+    def __init__(self, size: int, eps: float):
+        self.size, self.eps = size, eps
+        self.weight = self.bias = None
+
+    def param_specs(self):
+        return {"weight": ParamSpec((self.size,), role="scale"), "bias": ParamSpec((self.size,), role="scale")}
+
+    def prepare(self, device, act):
+        self.weight, self.bias = self.weight.float().contiguous(), self.bias.float().contiguous()
+
+    def over(self, inner) -> ops.NormedDelta:
+        return ops.NormedDelta(inner, self.weight, self.eps, bias=self.bias)
+
+    def forward(self, x, delta, ctx, rows=None, want_act=True, want_f32=False):
+        return ops.add_rmsnorm(x, delta, self.weight, self.eps, ctx.act, rows=rows, want_act=want_act, want_f32=want_f32,
+                               bias=self.bias)
