@@ -42,6 +42,12 @@ does it for the Gokezen design (mixer and feed-forward side by side behind one n
 with exponential gates; dense gated feed-forwards and clamped experts with a shared one, chosen by sigmoid scores within
 groups, in turn; a vector added before a looped pass) beside Qwen2-MoE with dense feed-forwards and experts with a shared one
 in turn.  A layer of the design has the memory's matrices over those of the layer beside it.
+
+    python bench.py --design pumozen [--design-sizes small,medium] [--layers 8]
+
+does it for the Pumozen design (a layer norm on every part's output only; attention normed over all heads whose values are its
+keys, differential attention, Mamba-2; clamped pairs and experts; a vector per token and layer) beside Qwen2-MoE with dense
+feed-forwards and experts with a shared one in turn.
 """
 from __future__ import annotations
 
@@ -387,6 +393,32 @@ def gokezen_config(z: dict, layers: int, max_positions: int) -> dict:
             "layers": [{"type": "parallel", "mixer": mixer, "mlp": moe if i % 2 else dense} for i in range(layers)]}
 
 
+def pumozen_config(z: dict, layers: int, max_positions: int) -> dict:
+    """`layers` layers in the order attention (norm over all heads, values that are the keys), differential attention, Mamba-2,
+    differential attention on that layer's keys and values; dense clamped pairs and routed experts with a gated shared one in
+    turn; a vector of a sixteenth of the width per token and layer.  A map of the differential attention is half as wide as a
+    head (two maps and their values are a head each); the state space has twice the width in heads of half a head, with a state
+    of 128 channels and one group."""
+    H, G, D, W = z["heads"], z["kv_heads"], z["dim"], z["width"]
+    dense = {"kind": "dense", "ff": z["dense_ff"], "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"], "limit": 7.0}, "shared": {"ff": z["ff"], "limit": 7.0},
+           "router": {"experts": z["experts"], "top": z["top"], "scale": 1.5}}
+    diff = {"heads": H, "kv_heads": G, "dim": D // 2, "vdim": D, "scale": (D // 2) ** -0.5, "diff": 0.6,
+            "q_temp": {"coef": 0.1, "every": 1024}}
+    kinds = [
+        ("attention", {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "rot": {"dims": D, "base": 1e4}}, dense),
+        ("attention_2", diff, moe),
+        ("mamba2", {"heads": 4 * W // D, "vdim": D // 2, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}, dense),
+        ("attention_2", diff, moe),
+    ]
+    out = []
+    for i in range(layers):
+        kind, mixer, mlp = kinds[i % 4]
+        out.append({"type": kind, "mixer": dict(mixer, kv_from=i - 2) if i % 4 == 3 else dict(mixer), "mlp": mlp})
+    return {"architecture": "Pumozen", "vocab": z["vocab"], "width": W, "norm": {"eps": 1e-5}, "token_side": {"dim": W // 16},
+            "layers": out}
+
+
 def qwen_mixed_shared_config_like(z: dict, layers: int, max_positions: int) -> dict:
     """The mixed layers with a shared expert as wide as a routed one beside the routed experts."""
     return dict(qwen_mixed_config_like(z, layers, max_positions), shared_expert_intermediate_size=z["ff"])
@@ -418,7 +450,8 @@ def design_comparison(args) -> int:
               "taminex": ("Taminex", taminex_config, qwen_dense_config_like),
               "beronex": ("Beronex", beronex_config, qwen_mixed_config_like),
               "bosalix": ("Bosalix", bosalix_config, qwen_config_like),
-              "gokezen": ("Gokezen", gokezen_config, qwen_mixed_shared_config_like)}[args.design]
+              "gokezen": ("Gokezen", gokezen_config, qwen_mixed_shared_config_like),
+              "pumozen": ("Pumozen", pumozen_config, qwen_mixed_shared_config_like)}[args.design]
     out = {"metric": f"{design[0]} beside Qwen2-MoE at equal sizes: prompt and decode tok/s, and milliseconds by kernel",
            "unit": "tok/s", "dtype": short, "layer_runs": layers, "data": "synthetic", "sizes": {}}
 
@@ -522,7 +555,7 @@ def main() -> int:
     ap.add_argument("--seed", type=int, default=None)
     ap.add_argument("--no-workloads", action="store_true",
                     help="leave out the two workloads of unequal prompts that the default run adds under \"workloads\"")
-    ap.add_argument("--design", default=None, choices=["felepel", "taminex", "beronex", "bosalix", "gokezen"],
+    ap.add_argument("--design", default=None, choices=["felepel", "taminex", "beronex", "bosalix", "gokezen", "pumozen"],
                     help="time this design beside Qwen2-MoE at equal sizes instead of the default workload")
     ap.add_argument("--design-sizes", default="small,medium", help="of " + ", ".join(DESIGN_SIZES))
     args = ap.parse_args()
