@@ -66,6 +66,15 @@ struct AttnArgs {
   int64_t ldo;                  // numbers between the rows of two tokens in out (nh * hd, or more for columns of a wider matrix)
 };
 
+// Differential attention: a head attends with two maps, whose keys are the two halves of a key row, to the same values; what is
+// left is r = a1 - lambda a2, divided by its root mean square over the values' vd numbers, times post, times sigmoid(gate).
+struct DiffArgs {
+  float lambda, eps, post;
+  int vd;
+  const float* gate;            // null, or [T][ld_gate] with nh * hd numbers a row
+  int64_t ld_gate;
+};
+
 // What softmax_tile needs of the score's changes for the QG groups of columns a lane holds: the plain scale, the cap and
 // each column's pair of the distance bias (a column is a token of one head in prompts, a head in decoding).
 template <int QG, bool MOD>
@@ -255,7 +264,8 @@ __device__ __forceinline__ void softmax_tile(f32x4 (&s)[QG][4], f32x4 (&o)[QG][D
 // exp(s * scale - max) with one instruction for the power.
 // VD, dt0: the wave sums the VD blocks of 16 value dimensions from block dt0 on (all DT of them unless a step's waves
 // share a head's value dimensions among them); the scores are over all of hd either way.
-template <int DT, int QG, bool EXACT, bool SWZ = false, bool ONCE = false, bool MOD = false, int VD = DT>
+// DIFF: groups of even number are columns of map 1, whose keys are the first half of a row, those of odd number of map 2.
+template <int DT, int QG, bool EXACT, bool SWZ = false, bool ONCE = false, bool MOD = false, int VD = DT, bool DIFF = false>
 __device__ __forceinline__ void tile_step(f32x4 (&o)[QG][VD], float (&m_run)[QG], float (&l_run)[QG],
                                           const bf16x8 (&qf)[QG][(DT + 1) / 2], const bf16_t* kt, int k_stride,
                                           const bf16_t* vt, int v_stride, int hd, int pos0, const int (&p_q)[QG],
@@ -301,7 +311,9 @@ __device__ __forceinline__ void tile_step(f32x4 (&o)[QG][VD], float (&m_run)[QG]
         const bf16x8 kf = SWZ ? ld16(kt + k_swz<DT>(krow, 4 * ks + c))
                               : (EXACT || d0 < hd ? ld16(kt + krow * k_stride + d0) : zero16());
 #pragma unroll
-        for (int g = 0; g < QG; ++g) s[g][jt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[g][ks], s[g][jt], 0, 0, 0);
+        for (int g = 0; g < QG; ++g)
+          if (!(DIFF && EXACT) || (ks < KS / 2) == (g % 2 == 0))      // (where the halves do not fall between steps, queries have zeros)
+            s[g][jt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[g][ks], s[g][jt], 0, 0, 0);
       }
     }
   }
@@ -441,12 +453,12 @@ __device__ __forceinline__ void attend_ahead(f32x4 (&o)[1][DT], float (&m_run)[1
 }
 
 template <int DT>
-__device__ __forceinline__ void load_query(bf16x8 (&qf)[(DT + 1) / 2], const bf16_t* qrow, int hd, bool valid) {
+__device__ __forceinline__ void load_query(bf16x8 (&qf)[(DT + 1) / 2], const bf16_t* qrow, int hd, bool valid, int from = 0) {
   const int c = (threadIdx.x % 64) / 16;
 #pragma unroll
   for (int ks = 0; ks < (DT + 1) / 2; ++ks) {
     const int d0 = 32 * ks + 8 * c;
-    qf[ks] = valid && d0 < hd ? ld16(qrow + d0) : zero16();
+    qf[ks] = valid && d0 >= from && d0 < hd ? ld16(qrow + d0) : zero16();      // (zeros in front of `from` and behind hd)
   }
 }
 
@@ -468,11 +480,13 @@ __device__ __forceinline__ void load_query(bf16x8 (&qf)[(DT + 1) / 2], const bf1
 // alone are 128 registers; the next tile still travels from memory into registers while this one is worked on.
 // VD < DT: the values' first 16 VD dimensions alone are summed and written (zeros behind them up to hd): an attention
 // whose keys are wider than its values, laid out at the keys' width.
-template <int DT, int QG, bool EXACT, bool MOD, int VD = DT>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > 16 ? 1 : 2))) void attn_prefill_kernel(AttnArgs a, int n_blocks, int B) {
+// DIFF: two maps a head, a token's two columns in two groups of one lane; they are made one where the output is normalised.
+template <int DT, int QG, bool EXACT, bool MOD, int VD = DT, bool DIFF = false>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > (DIFF ? 8 : 16) ? 1 : 2))) void attn_prefill_kernel(AttnArgs a, int n_blocks, int B, DiffArgs df) {
   constexpr bool ONEBUF = DT > ATTN_TWO_BUFFERS_UP_TO;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
-  constexpr int QW = 16 * QG;
+  static_assert(!DIFF || (QG % 2 == 0 && !MOD && VD == DT), "two maps a head: in pairs of groups, with plain scores");
+  constexpr int QW = 16 * (DIFF ? QG / 2 : QG);
   constexpr int KCH = (TILE * 2 * DT + 255) / 256;      // 16-byte chunks of a key tile per thread
   constexpr int VCH = (16 * VD * 8 + 255) / 256;        // and of a value tile
   static_assert(VD <= DT && (VD == DT || EXACT), "fewer value dimensions than key dimensions: for exact head sizes");
@@ -500,11 +514,12 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > 16 ? 1
   float m_run[QG], l_run[QG];
 #pragma unroll
   for (int g = 0; g < QG; ++g) {
-    const int qi = qb + wave * QW + g * 16 + r;
+    const int qi = qb + wave * QW + (DIFF ? g / 2 : g) * 16 + r;
     const bool valid = qi < n;
     p_q[g] = valid ? start + qi : -1;
     lo_q[g] = reach_lo(p_q[g], a.window, a.mod.chunk);
-    load_query<DT>(qf[g], a.q + ((size_t)(t0 + (valid ? qi : 0)) * a.nh + h) * hd, hd, valid);
+    load_query<DT>(qf[g], a.q + ((size_t)(t0 + (valid ? qi : 0)) * a.nh + h) * hd, DIFF && g % 2 == 0 ? hd / 2 : hd, valid,
+                   DIFF && g % 2 ? hd / 2 : 0);
 #pragma unroll
     for (int dt = 0; dt < VD; ++dt) o[g][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
     m_run[g] = -INFINITY;
@@ -587,7 +602,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > 16 ? 1
       if ((tile >= wave_beg || tile < kept) && tile < wave_end) {
         const int pos0 = tile * TILE;
         const bool masked = pos0 + TILE - 1 > wave_first || pos0 < wave_lo_last;
-        tile_step<DT, QG, EXACT, EXACT, false, MOD, VD>(o, m_run, l_run, qf, Ks, kstr, Vs, vstr, hd, pos0, p_q, lo_q,
+        tile_step<DT, QG, EXACT, EXACT, false, MOD, VD, DIFF>(o, m_run, l_run, qf, Ks, kstr, Vs, vstr, hd, pos0, p_q, lo_q,
                                         a.scale * LOG2E, masked, cm);
       }
       __syncthreads();
@@ -606,7 +621,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > 16 ? 1
     if ((tile >= wave_beg || tile < kept) && tile < wave_end) {
       const int pos0 = tile * TILE;
       const bool masked = pos0 + TILE - 1 > wave_first || pos0 < wave_lo_last;
-      tile_step<DT, QG, EXACT, EXACT, false, MOD, VD>(o, m_run, l_run, qf, Ks + cur, kstr, Vs + cur, vstr, hd, pos0, p_q, lo_q,
+      tile_step<DT, QG, EXACT, EXACT, false, MOD, VD, DIFF>(o, m_run, l_run, qf, Ks + cur, kstr, Vs + cur, vstr, hd, pos0, p_q, lo_q,
                                       a.scale * LOG2E, masked, cm);
     }
     __syncthreads();
@@ -614,6 +629,41 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DT > 16 ? 1
   }
 #undef TQ_FETCH
 #undef TQ_STAGE
+  if constexpr (DIFF) {
+#pragma unroll
+    for (int g = 0; g < QG; g += 2) {
+      const float i1 = 1.0f / l_run[g], i2 = -df.lambda / l_run[g + 1];
+      float ss = 0.f;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt)
+        if (16 * dt < hd)
+#pragma unroll
+          for (int v = 0; v < 4; ++v) {
+            const float x = fmaf(o[g][dt][v], i1, o[g + 1][dt][v] * i2);
+            o[g][dt][v] = x;
+            ss = fmaf(x, x, ss);
+          }
+      ss = group_sum(ss);      // (before lanes without a token leave: the four lanes of a column have it or not together)
+      if (p_q[g] < 0) continue;
+      const float f = df.post / sqrtf(ss / (float)df.vd + df.eps);
+      const size_t t = t0 + p_q[g] - start;
+      bf16_t* orow = a.out + t * a.ldo + (size_t)h * hd;
+      const float* gr = df.gate ? df.gate + t * df.ld_gate + (size_t)h * hd : nullptr;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) {
+        if (16 * dt < hd) {
+          f32x4 x = o[g][dt] * f;
+          if (gr) {
+            const f32x4 z = *reinterpret_cast<const f32x4*>(gr + 16 * dt + 4 * c);
+#pragma unroll
+            for (int v = 0; v < 4; ++v) x[v] /= 1.0f + expf(-z[v]);
+          }
+          *reinterpret_cast<u32x2*>(orow + 16 * dt + 4 * c) = u32x2{pack2(x[0], x[1]), pack2(x[2], x[3])};
+        }
+      }
+    }
+    return;
+  }
 #pragma unroll
   for (int g = 0; g < QG; ++g) {
     if (p_q[g] < 0) continue;
@@ -774,6 +824,79 @@ __global__ __launch_bounds__(256) void attn_join_kernel(AttnArgs a) {
 #undef RUN_OF
 }
 
+// The same for two maps a head: a.nh counts the maps' columns (head h's maps are 2 h and 2 h + 1), grid (nh / 2, B), block 128:
+// a wave joins a map's runs, then the first makes the two one.  A lane takes NP pairs of neighbouring dimensions (heads of up
+// to 128 NP; every load is unconditional, from an address clamped into the row).
+template <int NP>
+__global__ __launch_bounds__(128) void attn_join_diff_kernel(AttnArgs a, DiffArgs df) {
+  extern __shared__ float wgt_all[];        // [2][MAX_RUNS_LDS]
+  __shared__ float other[128 * NP];
+  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x % 64, map = threadIdx.x / 64;
+  float* wgt = wgt_all + map * MAX_RUNS_LDS;
+  const int n_runs = a.start[b] / TILE / tiles_per_run(a.start[b]) + 1, stride = a.hd + 2;
+  const float* part = a.partial + ((size_t)b * a.nh + 2 * h + map) * a.max_runs * stride;
+  float m = -INFINITY;
+  for (int i = lane; i < n_runs; i += 64) m = fmaxf(m, part[(size_t)i * stride + a.hd]);
+  m = wave_max(m);
+  float l = 0.f;
+  for (int i0 = 0; i0 < n_runs; i0 += 64) {
+    const int i = i0 + lane;
+    float w = 0.f, wl = 0.f;
+    if (i < n_runs) {
+      w = __builtin_amdgcn_exp2f(part[(size_t)i * stride + a.hd] - m);
+      wl = w * part[(size_t)i * stride + a.hd + 1];
+      wgt[i] = w;
+    }
+    l += wave_sum(wl);
+  }
+  __builtin_amdgcn_wave_barrier();
+  const float inv = 1.0f / l;
+  float2 acc[NP];
+  int at[NP];
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    acc[j] = float2{0.f, 0.f};
+    at[j] = min(128 * j + 2 * lane, a.hd - 2);
+  }
+#pragma unroll 8
+  for (int i = 0; i < n_runs; ++i) {
+#pragma unroll
+    for (int j = 0; j < NP; ++j) {
+      const float2 v = *reinterpret_cast<const float2*>(part + (size_t)i * stride + at[j]);
+      acc[j].x = fmaf(wgt[i], v.x, acc[j].x);
+      acc[j].y = fmaf(wgt[i], v.y, acc[j].y);
+    }
+  }
+  if (map == 1)
+#pragma unroll
+    for (int j = 0; j < NP; ++j) {
+      other[128 * j + 2 * lane] = acc[j].x * inv;
+      other[128 * j + 2 * lane + 1] = acc[j].y * inv;
+    }
+  __syncthreads();
+  if (map == 1) return;
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const bool has = 128 * j + 2 * lane < a.hd;
+    acc[j].x = has ? fmaf(acc[j].x, inv, -df.lambda * other[128 * j + 2 * lane]) : 0.f;
+    acc[j].y = has ? fmaf(acc[j].y, inv, -df.lambda * other[128 * j + 2 * lane + 1]) : 0.f;
+    ss = fmaf(acc[j].x, acc[j].x, fmaf(acc[j].y, acc[j].y, ss));
+  }
+  const float f = df.post / sqrtf(wave_sum(ss) / (float)df.vd + df.eps);
+  const size_t t = a.cu_seqlens[b];
+  bf16_t* orow = a.out + t * a.ldo + (size_t)h * a.hd;
+  const float* gr = df.gate ? df.gate + t * df.ld_gate + (size_t)h * a.hd : nullptr;
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    if (128 * j + 2 * lane < a.hd) {
+      const float2 z = gr ? *reinterpret_cast<const float2*>(gr + at[j]) : float2{0.f, 0.f};
+      const float gx = gr ? 1.0f / (1.0f + expf(-z.x)) : 1.0f, gy = gr ? 1.0f / (1.0f + expf(-z.y)) : 1.0f;
+      *reinterpret_cast<uint32_t*>(orow + at[j]) = pack2(acc[j].x * f * gx, acc[j].y * f * gy);
+    }
+  }
+}
+
 // ------------------------------------------------------------------------------------------ launch
 template <int DT, int QG, bool EXACT, bool MOD, int VD = DT>
 static int launch_prefill_as(const AttnArgs& a, int B, int max_new, hipStream_t st) {
@@ -782,7 +905,7 @@ static int launch_prefill_as(const AttnArgs& a, int B, int max_new, hipStream_t 
     (void)hipFuncSetAttribute((const void*)attn_prefill_kernel<DT, QG, EXACT, MOD, VD>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem);
   const int n_blocks = (max_new + 64 * QG - 1) / (64 * QG);
   if ((int64_t)n_blocks * a.nh * B > 0x7fffffff) return TQ_ERR_UNSUPPORTED;
-  hipLaunchKernelGGL((attn_prefill_kernel<DT, QG, EXACT, MOD, VD>), dim3(n_blocks * a.nh * B), dim3(256), shmem, st, a, n_blocks, B);
+  hipLaunchKernelGGL((attn_prefill_kernel<DT, QG, EXACT, MOD, VD>), dim3(n_blocks * a.nh * B), dim3(256), shmem, st, a, n_blocks, B, DiffArgs{});
   return 0;
 }
 // (the kernels that cap or bias scores are instantiations of their own, so that the others carry nothing of it)
@@ -792,7 +915,7 @@ static int launch_prefill(const AttnArgs& a, int B, int max_new, hipStream_t st)
                                        : launch_prefill_as<DT, QG, EXACT, false, VD>(a, B, max_new, st);
 }
 template <int DT, bool EXACT, bool MOD>
-static void launch_decode_as(const AttnArgs& a, int B, int grid_runs, hipStream_t st) {
+static void launch_decode_as(const AttnArgs& a, int B, int grid_runs, hipStream_t st, const DiffArgs* df = nullptr) {
   const int g = a.nh / a.nkv;
   const dim3 join_block(a.hd % 128 == 0 ? 64 * (a.hd / 128) : 64);      // a wave to every 128 dimensions of a head
   if constexpr (DT > 16) {
@@ -806,12 +929,29 @@ static void launch_decode_as(const AttnArgs& a, int B, int grid_runs, hipStream_
     else
       hipLaunchKernelGGL((attn_decode_kernel<DT, EXACT, false, MOD>), grid, dim3(64), 0, st, a);
   }
-  hipLaunchKernelGGL(attn_join_kernel, dim3(a.nh, B), join_block, join_block.x / 64 * MAX_RUNS_LDS * sizeof(float), st, a);
+  if (df && a.hd <= 128)
+    hipLaunchKernelGGL(attn_join_diff_kernel<1>, dim3(a.nh / 2, B), dim3(128), 2 * MAX_RUNS_LDS * sizeof(float), st, a, *df);
+  else if (df)
+    hipLaunchKernelGGL(attn_join_diff_kernel<2>, dim3(a.nh / 2, B), dim3(128), 2 * MAX_RUNS_LDS * sizeof(float), st, a, *df);
+  else
+    hipLaunchKernelGGL(attn_join_kernel, dim3(a.nh, B), join_block, join_block.x / 64 * MAX_RUNS_LDS * sizeof(float), st, a);
 }
 template <int DT, bool EXACT>
 static void launch_decode(const AttnArgs& a, int B, int grid_runs, hipStream_t st) {
   if (a.mod.cap > 0.f || a.mod.r1 || a.mod.pb || a.mod.keep > 0) launch_decode_as<DT, EXACT, true>(a, B, grid_runs, st);
   else launch_decode_as<DT, EXACT, false>(a, B, grid_runs, st);
+}
+
+// Two maps a head.  Prompts: 16 tokens with both their maps to a wave.
+template <int DT, bool EXACT>
+static int launch_diff_prefill(const AttnArgs& a, const DiffArgs& df, int B, int max_new, hipStream_t st) {
+  const size_t shmem = (DT > ATTN_TWO_BUFFERS_UP_TO ? 1 : 2) * (EXACT ? (size_t)TILE * (a.hd + 16 * DT) : (size_t)TILE * (a.hd + KPAD) + (size_t)a.hd * VSTR) * sizeof(bf16_t);
+  if (shmem > 48 * 1024)
+    (void)hipFuncSetAttribute((const void*)attn_prefill_kernel<DT, 2, EXACT, false, DT, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem);
+  const int n_blocks = (max_new + 63) / 64;
+  if ((int64_t)n_blocks * a.nh * B > 0x7fffffff) return TQ_ERR_UNSUPPORTED;
+  hipLaunchKernelGGL((attn_prefill_kernel<DT, 2, EXACT, false, DT, true>), dim3(n_blocks * a.nh * B), dim3(256), shmem, st, a, n_blocks, B, df);
+  return 0;
 }
 
 // Number of floats of `partial` that decoding B sequences up to position max_end needs.
@@ -922,4 +1062,46 @@ TQ_API int tq_attention_mfma(const void* q, const void* k_pool, const void* v_po
   return tq_attention_mfma_mod(q, k_pool, v_pool, block_table, bt_stride, cu_seqlens, slots, start, page_size, page_stride,
                                B, nh, nkv, hd, window, scale, 0.f, nullptr, nullptr, 0, nullptr, out, partial, decode, max_new,
                                max_end, st);
+}
+
+// Differential attention over heads of hd (a multiple of 32, at most 256): a key row holds both maps' keys, each half of hd wide,
+// a value row hd numbers of which the first vd count.  Prompts: q [T][nh][hd], both maps of a head side by side; decoding:
+// q [T][2 nh][hd], each map alone with zeros in the other's place.  out [T][nh][hd] = r / sqrt(sum(r^2) / vd + eps) * post *
+// sigmoid(gate), r = a1 - lambda a2; gate: float rows ld_gate apart, or null.  partial as tq_attention_decode_scratch says for 2 nh
+// heads.
+TQ_API int tq_attention_mfma_diff(const void* q, const void* k_pool, const void* v_pool, const int* block_table, int bt_stride,
+                                  const int* cu_seqlens, const int* slots, const int* start, int page_size, int64_t page_stride,
+                                  int B, int nh, int nkv, int hd, float scale, float lambda, float eps, int vd, float post,
+                                  const float* gate, int64_t ld_gate, void* out, float* partial, int decode, int max_new,
+                                  int max_end, hipStream_t st) {
+  if (B <= 0) return 0;
+  if (hd % 32 != 0 || hd < 32 || hd > 256 || page_size % TILE != 0 || nkv <= 0 || nh % nkv != 0) return TQ_ERR_UNSUPPORTED;
+  if (nh > 32767 || B > 65535 || page_stride % 8 != 0 || !(scale > 0.f)) return TQ_ERR_UNSUPPORTED;
+  if (vd < 1 || vd > hd || (gate && (ld_gate < (int64_t)nh * hd || ld_gate % 4 != 0 || (uintptr_t)gate % 16 != 0))) return TQ_ERR_BAD_ARG;
+  if (decode && (!partial || most_runs(max_end) > MAX_RUNS_LDS)) return TQ_ERR_BAD_ARG;
+  const DiffArgs df{lambda, eps, post, vd, gate, ld_gate};
+  AttnArgs a{(const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_table, bt_stride, cu_seqlens, slots,
+             start, page_size, page_stride, decode ? 2 * nh : nh, nkv, hd, 0, scale, (bf16_t*)out, partial,
+             most_runs(max_end), ScoreMod{}, nullptr, 0, (int64_t)nh * hd};
+  const int dt = hd / 16;
+  int rc = 0;
+  if (decode) {
+    const int grid_runs = runs_at(max_end > 0 ? max_end - 1 : 0);
+    if (dt == 4) launch_decode_as<4, true, false>(a, B, grid_runs, st, &df);
+    else if (dt == 8) launch_decode_as<8, true, false>(a, B, grid_runs, st, &df);
+    else if (dt == 16) launch_decode_as<16, true, false>(a, B, grid_runs, st, &df);
+    else if (dt < 4) launch_decode_as<4, false, false>(a, B, grid_runs, st, &df);
+    else if (dt < 8) launch_decode_as<8, false, false>(a, B, grid_runs, st, &df);
+    else launch_decode_as<16, false, false>(a, B, grid_runs, st, &df);
+  } else {
+    if (dt == 4) rc = launch_diff_prefill<4, true>(a, df, B, max_new, st);
+    else if (dt == 8) rc = launch_diff_prefill<8, true>(a, df, B, max_new, st);
+    else if (dt == 16) rc = launch_diff_prefill<16, true>(a, df, B, max_new, st);
+    else if (dt < 4) rc = launch_diff_prefill<4, false>(a, df, B, max_new, st);
+    else if (dt < 8) rc = launch_diff_prefill<8, false>(a, df, B, max_new, st);
+    else rc = launch_diff_prefill<16, false>(a, df, B, max_new, st);
+  }
+  if (rc) return rc;
+  TQ_LAUNCH_CHECK();
+  return 0;
 }

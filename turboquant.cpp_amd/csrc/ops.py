@@ -127,6 +127,7 @@ _SIGNATURES = {
     "tq_add_norm": [_c_ptr, _c_ptr, _c_int, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_f32,
                     _c_int, _c_ptr, _c_ptr, _c_f32, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
     "tq_token_gate": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
+    "tq_token_gate_product": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "tq_row_norm_kv_write": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_f32, _c_ptr, _c_ptr,
                              _c_int, _c_f32, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_int,
                              _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
@@ -190,6 +191,9 @@ _OPTIONAL = {
     "tq_attention_mfma_ld": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int,
                              _c_int, _c_int, _c_int, _c_int, _c_f32, _c_f32, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                              _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_int, _c_i64, _c_ptr],
+    "tq_attention_mfma_diff": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_int,
+                               _c_int, _c_int, _c_f32, _c_f32, _c_f32, _c_int, _c_f32, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int,
+                               _c_int, _c_int, _c_ptr],
     "tq_attention_mfma_mod": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_i64, _c_int, _c_int,
                               _c_int, _c_int, _c_int, _c_f32, _c_f32, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
                               _c_int, _c_int, _c_ptr],
@@ -2153,6 +2157,27 @@ def token_gate(p: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, activ
     return out
 
 
+def token_gate_product(a: torch.Tensor, w: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, activation: str, act) -> torch.Tensor:
+    """``token_gate`` of the product a w^T (``w`` [N, K]): one launch for up to 16 tokens, else two."""
+    k = "token_gate_product"
+    adt = ACT_DTYPES[dtype_name(act)]
+    T, K = a.shape
+    if (T > 16 or w.dtype != adt or a.dtype != adt or K % (16 // adt.itemsize) or a.stride(0) % (16 // adt.itemsize)
+            or a.data_ptr() % 16 or w.data_ptr() % 16):
+        return token_gate(gemm(a, w, act, partial_sums=True), tokens, table, activation, act)
+    _need(a.is_cuda and a.stride(1) == 1, k, "a must be on the GPU with unit stride along its rows")
+    _check(w, k, "w", adt)
+    N = w.shape[0]
+    _need(w.dim() == 2 and w.shape[1] == K, k, lambda: f"w must be [N, {K}]")
+    _check(tokens, k, "tokens", torch.int32, (T,))
+    _need(isinstance(table, torch.Tensor) and table.is_cuda and table.dtype in _WTYPE and table.dim() == 2 and table.shape[1] == N
+          and table.stride(1) == 1, k, lambda: f"table must be [V, {N}] on the GPU with unit stride along its rows")
+    out = torch.empty((T, N), dtype=adt, device=a.device)
+    _run(k, library(act).tq_token_gate_product(_ptr(a), a.stride(0), _ptr(w), _ptr(tokens), _ptr(table), _WTYPE[table.dtype],
+                                               table.stride(0), _gate_code(k, activation), _ptr(out), T, N, K, _stream()))
+    return out
+
+
 # ------------------------------------------------------------------ between a product and its attention
 def _kv_places(k: str, k_pages, v_pages, layer_offset: int, page_size: int, page_stride: int, num_kv_heads: int, head_dim: int,
                block_table, runs, adt):
@@ -2255,6 +2280,59 @@ def diff_prep_kv_write(qkv: torch.Tensor, positions: torch.Tensor, seq_of_token:
         *places, page_size, page_stride, T, num_heads, num_kv_heads if write else 0, head_dim, int(write), int(expand), *tiles,
         _stream()))
     return q
+
+
+def diff_attention_fused(act, head_dim: int, page_size: int, page_stride: int, scale: float) -> bool:
+    """Whether ``diff_attention`` runs both maps of a head in one pass over keys and values (else two heads to a head's maps)."""
+    return (dtype_name(act) == "bfloat16" and has_kernel(act, "tq_attention_mfma_diff") and head_dim % 32 == 0 and head_dim <= 256
+            and page_size % 64 == 0 and page_stride % 8 == 0 and scale > 0)
+
+
+def diff_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, layer_offset: int, positions: torch.Tensor,
+                   seq_of_token: torch.Tensor, block_table: torch.Tensor, page_size: int, page_stride: int, num_heads: int,
+                   num_kv_heads: int, head_dim: int, scale: float, lam: float, eps: float, value_dim: int, post: float,
+                   gate: torch.Tensor | None, act, runs: dict) -> torch.Tensor:
+    """Differential attention behind ``diff_prep_kv_write``: both maps of every head over the cached rows, and ``diff_combine`` of
+    what they leave; [T, nh * hd].  ``q`` as ``diff_prep_kv_write`` returns it: expanded, except where
+    ``diff_attention_fused`` and the step is no decode step."""
+    k = "diff_attention"
+    T = positions.numel()
+    if not diff_attention_fused(act, head_dim, page_size, page_stride, scale):
+        o = attention(q, k_pages, v_pages, layer_offset, positions, seq_of_token, block_table, page_size, page_stride, 2 * num_heads,
+                      num_kv_heads, head_dim, None, scale, act, runs=runs)
+        return diff_combine(o, lam, eps, value_dim, post, gate, num_heads, head_dim, act)
+    adt, lib = ACT_DTYPES[dtype_name(act)], library(act)
+    decode = bool(runs["decode"])
+    N = num_heads * head_dim
+    _check(q, k, "q", adt, (T, (2 if decode else 1) * N))
+    _check(k_pages, k, "k_pages", adt)
+    _check(v_pages, k, "v_pages", adt)
+    _check(block_table, k, "block_table", torch.int32)
+    B = runs["slots"].numel()
+    _check(runs["cu_seqlens"], k, "cu_seqlens", torch.int32, (B + 1,))
+    _check(runs["slots"], k, "slots", torch.int32, (B,))
+    _check(runs["start"], k, "start", torch.int32, (B,))
+    _need(block_table.dim() == 2 and runs["max_end"] <= block_table.shape[1] * page_size, k, "positions reach beyond the page table")
+    _need(num_heads % num_kv_heads == 0 and layer_offset + num_kv_heads * page_size * head_dim <= page_stride, k,
+          "heads must be a multiple of kv heads, and the layer must fit in a page")
+    _need(1 <= value_dim <= head_dim, k, "the values' width lies within the head")
+    _need(gate is None or (gate.is_cuda and gate.dtype == torch.float32 and tuple(gate.shape) == (T, N) and gate.stride(1) == 1
+                           and gate.stride(0) % 4 == 0 and gate.data_ptr() % 16 == 0), k,
+          lambda: f"gate must be float32 [{T}, {N}] on the GPU, rows at multiples of 16 bytes")
+    partial = None
+    if decode:
+        _need(T == B, k, "decoding brings one token per sequence")
+        partial = torch.empty((lib.tq_attention_decode_scratch(B, 2 * num_heads, head_dim, int(runs["max_end"])),),
+                              dtype=torch.float32, device=q.device)
+    out = torch.empty((T, N), dtype=adt, device=q.device)
+    esz = k_pages.element_size()
+    _run("attention_mfma", lib.tq_attention_mfma_diff(
+        _ptr(q), k_pages.data_ptr() + layer_offset * esz, v_pages.data_ptr() + layer_offset * esz, _ptr(block_table),
+        block_table.shape[1], _ptr(runs["cu_seqlens"]), _ptr(runs["slots"]), _ptr(runs["start"]), page_size, page_stride, B, num_heads,
+        num_kv_heads, head_dim, float(scale), float(lam), float(eps), int(value_dim), float(post), _ptr(gate),
+        gate.stride(0) if gate is not None else 0, _ptr(out), _ptr(partial), int(decode), int(runs["max_new"]), int(runs["max_end"]),
+        _stream()))
+    return out
 
 
 def diff_combine(o: torch.Tensor, lam: float, eps: float, value_dim: int, post: float, gate: torch.Tensor | None, num_heads: int,

@@ -390,7 +390,7 @@ __global__ __launch_bounds__(256) void ssd_chunk_prefix_kernel(const int* __rest
   *srow = carry;
 }
 
-// grid (ceil(V / LC_V), H / hb, B * NC), block 256: a chunk's read-outs for LC_V value channels, a wave to 16 tokens.  (The
+// grid (ceil(V / LC_V), H / hb, B * NC), block 256: a chunk's read-outs for LC_V value channels.  (The
 // values wait in registers until B has been read and take its place in LDS: with states of up to 128 channels two workgroups
 // fit a compute unit.)
 template <int ND, bool VEC>
@@ -442,10 +442,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND > 8 ? 1 
       if (ct <= wave) sc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, ks[(16 * ct + r) * QLD + 4 * k4 + g], sc[ct], 0, 0, 0);
   }
   float* ps = ks;
+  // From here on a wave takes 16 value channels of all the chunk's tokens, so that it reads its columns of the state once.
+  // (Loads are unconditional, from addresses within the state: rows beyond N meet zeros of C, columns beyond V are not stored.)
+  const int v = v0 + 16 * wave + r, vl = min(v, V - 1);
+  const float* sb = scratch + ((size_t)gi * H + h0) * N * V + vl;
+  constexpr int AHEAD = DP / 4 > 32 ? 32 : DP / 4;
   for (int u = 0; u < hb; ++u) {
     const int h = h0 + u;
     const double* F = Fs + u * LC_T;
     const float* step = dts + u * LC_T;
+    float sv[AHEAD];
+#pragma unroll
+    for (int k4 = 0; k4 < AHEAD; ++k4) sv[k4] = sb[(size_t)min(4 * k4 + g, N - 1) * V];
     __syncthreads();                      // every wave has read B, or the scores and values of the head before
     vr_.store_turned(vs, tid);
 #pragma unroll
@@ -460,38 +468,44 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND > 8 ? 1 
     lc_f32x4 acc[4], far[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = far[i] = lc_f32x4{0.f, 0.f, 0.f, 0.f};
-    // what the state before the chunk adds: S^T C, each row times e^(F_t)
-    const float* sb = scratch + ((size_t)gi * H + h) * N * V + v0 + r;
-#pragma unroll 8
-    for (int k4 = 0; k4 < DP / 4; ++k4) {
-      const float a = qrow[4 * k4];
-      const int k = 4 * k4 + g;
+    // the chunk's own tokens: a tile of 16 of them reaches the tiles up to its own
 #pragma unroll
-      for (int cv = 0; cv < 4; ++cv) {
-        const float bv = k < N && v0 + 16 * cv + r < V ? sb[(size_t)k * V + 16 * cv] : 0.f;
-        far[cv] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, bv, far[cv], 0, 0, 0);
+    for (int ct = 0; ct < 4; ++ct)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const int k4 = 4 * ct + k;
+        const float bv = vs[(4 * k4 + g) * LC_V + ((16 * wave + r) ^ (16 * g))];
+#pragma unroll
+        for (int tt = 0; tt < 4; ++tt)
+          if (tt >= ct) acc[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ps[(16 * tt + r) * PLD + 4 * k4 + g], bv, acc[tt], 0, 0, 0);
       }
-    }
-    const float* prow = ps + (16 * wave + r) * PLD + g;
-    for (int k4 = 0; k4 < 4 * (wave + 1); ++k4) {
-      const float a = prow[4 * k4];
-      const float* vr = vs + (4 * k4 + g) * LC_V + r;
+    // what the state before the chunk adds: S^T C, each row times e^(F_t)
+    const float* qr = qs + r * QLD + g;
 #pragma unroll
-      for (int cv = 0; cv < 4; ++cv) acc[cv] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vr[16 * (cv ^ g)], acc[cv], 0, 0, 0);
+    for (int k4 = 0; k4 < AHEAD; ++k4)
+#pragma unroll
+      for (int tt = 0; tt < 4; ++tt)
+        far[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(qr[16 * tt * QLD + 4 * k4], sv[k4], far[tt], 0, 0, 0);
+#pragma unroll 8
+    for (int k4 = AHEAD; k4 < DP / 4; ++k4) {
+      const float bv = sb[(size_t)min(4 * k4 + g, N - 1) * V];
+#pragma unroll
+      for (int tt = 0; tt < 4; ++tt)
+        far[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(qr[16 * tt * QLD + 4 * k4], bv, far[tt], 0, 0, 0);
     }
     const float skip = Dh[h];
+    if (v < V)
 #pragma unroll
-    for (int cv = 0; cv < 4; ++cv) {
-      const int v = v0 + 16 * cv + r;
+      for (int tt = 0; tt < 4; ++tt)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = 16 * wave + 4 * g + i;
-        if (t < nc && v < V) {
-          const float x = vs[t * LC_V + ((16 * cv + r) ^ (16 * (t & 3)))];
-          y[((size_t)(t0 + c * LC_T + t) * H + h) * V + v] = fmaf(skip, x, fmaf(expf((float)F[t]), far[cv][i], acc[cv][i]));
+        for (int i = 0; i < 4; ++i) {
+          const int t = 16 * tt + 4 * g + i;
+          if (t < nc) {
+            const float x = vs[t * LC_V + ((16 * wave + r) ^ (16 * (t & 3)))];
+            y[((size_t)(t0 + c * LC_T + t) * H + h) * V + v] = fmaf(skip, x, fmaf(expf((float)F[t]), far[tt][i], acc[tt][i]));
+          }
         }
-      }
-    }
+    sb += (size_t)N * V;
   }
 }
 

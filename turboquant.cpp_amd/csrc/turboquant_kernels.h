@@ -218,6 +218,13 @@ int tq_add_norm(float* x, const float* delta, int S, int64_t delta_stride, const
         int H, hipStream_t st);
 int tq_token_gate(const float* p, int S, const int* tokens, const void* table, int wtype, int64_t ld_table, int kind,
         void* out, int T, int N, hipStream_t st);
+int tq_token_gate_product(const void* a, int64_t lda, const void* w, const int* tokens, const void* table, int wtype,
+        int64_t ld_table, int kind, void* out, int T, int N, int K, hipStream_t st);
+// attention_mfma.hip: two maps a head over one pass of keys and values (bfloat16 library)
+int tq_attention_mfma_diff(const void* q, const void* k_pool, const void* v_pool, const int* block_table, int bt_stride,
+        const int* cu_seqlens, const int* slots, const int* start, int page_size, int64_t page_stride, int B, int nh,
+        int nkv, int hd, float scale, float lambda, float eps, int vd, float post, const float* gate, int64_t ld_gate,
+        void* out, float* partial, int decode, int max_new, int max_end, hipStream_t st);
 // attention_prep.hip: between a product and its attention; two maps a head made one
 int tq_row_norm_kv_write(const float* qkv, int64_t ld, const int* positions, const int* seq_of_token,
         const int* block_table, int bt_stride, const float* inv_freq, int pairing, int rot, float amp, const void* wq,

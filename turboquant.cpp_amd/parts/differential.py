@@ -14,7 +14,8 @@ a head's output is ``o = a1 - lambda a2``, divided by its root mean square over 
 
 Layout: a key head's two maps lie side by side in one row of the cache, each ``D / 2`` wide, D being twice the larger of
 head_dim and half the value width rounded up to 16; the value row is D wide.  So both maps' scores come from one pass over one
-row of keys, and no value is kept twice.  Added rows and columns of the matrices are zeros.  Float32 on both libraries: norms,
+row of keys, and no value is kept twice.  On the bfloat16 library, for rows of up to 256, the difference, its norm and the gate
+are made where the attention normalises its output.  Added rows and columns of the matrices are zeros.  Float32 on both libraries: norms,
 temperature, scores, softmax, lambda, the difference's norm and the gate.
 """
 from __future__ import annotations
@@ -100,10 +101,13 @@ class DifferentialAttention(Part):
         H, G, D = self.num_heads, self.num_kv_heads, self.head_dim
         proj = ops.gemm(normed, self.in_weight, ctx.act)                   # float32 [T, q | k | v | gate], or [T, q | gate]
         width = (H + (0 if self.shares_kv else 2 * G)) * D
+        # queries: both maps of a head side by side where one pass over the keys serves both, else each map with zeros beside it
+        expand = b.is_decode or not ops.diff_attention_fused(ctx.act, D, kv.page_size, kv.page_stride, self.scale)
         q = ops.diff_prep_kv_write(proj[:, :width], b.positions, b.slot_of_token, kv.table, kv.k_pages if kv.owns else None,
                                    kv.v_pages if kv.owns else None, kv.layer_offset, kv.page_size, kv.page_stride, H, G, D, ctx.act,
-                                   self.q_norm, self.k_norm, self.eps, self.key_dim, self.temperature, runs=b.runs())
-        o = ops.attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table, kv.page_size,
-                          kv.page_stride, 2 * H, G, D, None, self.scale, ctx.act, runs=b.runs())
-        o = ops.diff_combine(o, self.lam, self.eps, self.value_dim, 1.0 - self.diff, proj[:, width:], H, D, ctx.act)
+                                   self.q_norm, self.k_norm, self.eps, self.key_dim, self.temperature, expand=expand,
+                                   runs=b.runs())
+        o = ops.diff_attention(q, kv.k_pages, kv.v_pages, kv.layer_offset, b.positions, b.slot_of_token, kv.table, kv.page_size,
+                               kv.page_stride, H, G, D, self.scale, self.lam, self.eps, self.value_dim, 1.0 - self.diff,
+                               proj[:, width:], ctx.act, b.runs())
         return ops.gemm(o, self.out_weight, ctx.act, partial_sums=True)

@@ -6,7 +6,7 @@
     x <- x + y / sqrt(mean(y^2) + eps) * weight
 
 f one of the activations of ``ops.GATES``.  Float32 on both libraries: the activation, its product with e, the norm.  Three
-launches: the product, ``token_gate``, the second product, whose partial sums the next norm adds up, norms and adds.
+launches (two for up to 16 tokens): the product, ``token_gate``, the second product, whose partial sums the next norm adds up, norms and adds.
 """
 from __future__ import annotations
 
@@ -34,6 +34,5 @@ class TokenSide(Part):
         self.norm = self.norm.float().contiguous()      # it enters float arithmetic only
 
     def forward(self, h, ctx) -> ops.NormedDelta:
-        p = ops.gemm(h, self.gate, ctx.act, partial_sums=True)
-        g = ops.token_gate(p, ctx.batch.tokens, self.token_rows, self.activation, ctx.act)
+        g = ops.token_gate_product(h, self.gate, ctx.batch.tokens, self.token_rows, self.activation, ctx.act)
         return ops.NormedDelta(ops.gemm(g, self.proj, ctx.act, partial_sums=True), self.norm, self.eps)
