@@ -686,7 +686,7 @@ def test_norm_and_position_parts_alone(act):
     with pytest.raises(ValueError, match="pairing"):
         build_part("position", PartSpec("rope", dict(head_dim=8, rotary_dim=8, theta=1.0, pairing="odd")))
     with pytest.raises(ValueError, match="unknown norm"):
-        build_part("norm", PartSpec("layernorm", {}))
+        build_part("norm", PartSpec("no_such_norm", {}))
 
 
 # ------------------------------------------------------------------------------------------------ a toy mixer with state
