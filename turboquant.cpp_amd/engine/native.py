@@ -28,6 +28,8 @@ class NativeModel:
             raise ValueError("the step executor embeds tokens without a learned vector per position")
         if getattr(model, "step_vectors", None) is not None:
             raise ValueError("the step executor adds no vectors between layers")
+        if getattr(model, "token_table", None) is not None:
+            raise ValueError("the step executor knows no second table with a row per token")
         if model.plan.logit_scale != 1.0:
             raise ValueError("the step executor does not multiply its logits by a constant")
         layers = [b.native() for b in model.blocks]
